@@ -2,7 +2,7 @@
 layer with the xIELU activation, a mixture of small experts chosen by a
 per-token-id table (no learned router at run time), a gated dense layer with
 the tanh form of gelu, and a mixture of clamped gated experts chosen by a
-learned router."""
+learned router, the weights on their outputs or their inputs."""
 from __future__ import annotations
 
 import math
@@ -28,8 +28,11 @@ class FFCfg:
     act: str = "clamp"
     # "top": weights = softmax over the chosen logits; "all": scores =
     # softmax over all logits, the chosen scores divided by their sum and
-    # multiplied by route_scale
+    # multiplied by route_scale; "sigmoid": every logit's own sigmoid times
+    # route_scale, not renormalised
     score: str = "top"
+    # the weights multiply the experts' inputs instead of their outputs
+    weigh_input: bool = False
     groups: int = 0          # experts in this many equal runs of neighbours,
     keep: int = 0            # of which only the best `keep` can be chosen
     route_scale: float = 1.0
@@ -200,18 +203,20 @@ class RoutedMoE(nn.Module):
     Variants by configuration: experts of the form down(silu(gate h) up h)
     (`act`); scores from a softmax over ALL logits, the chosen ones divided
     by their sum and scaled, the choice limited to the best `keep` of
-    `groups` runs of neighbouring experts (`score`, `groups`); an always-on
-    shared expert of the same form (`shared_ff`), which enters the fold as
-    one more chosen row with weight 1. Weights are stacked [E, 2 ff', W] (gate rows,
-    then up rows, each padded to a multiple of 8) and [E, W, ff].
+    `groups` runs of neighbouring experts (`score`, `groups`); scores that
+    are each logit's own sigmoid, used as they are (`score`); weights on the
+    experts' inputs, act(w gate h) * (w up h), where they enter as a factor
+    of the two products in fp32 (`weigh_input`); an always-on shared expert
+    of the same form (`shared_ff`), added with weight 1. Weights are stacked
+    [E, 2 ff', W] (gate rows, then up rows, each padded to a multiple of 8)
+    and [E, W, ff].
 
     Two forms behind one call. Few rows (decode steps; nothing leaves the
-    device, so the step can sit in a captured graph): every expert runs on
-    every row as one batched GEMM pair — a batch of a few dozen rows
-    touches nearly every expert anyway, so the weights stream once — and
-    the fold picks each row's chosen results. Many rows (prompt portions):
-    the (row, expert) pairs are sorted by expert, the group sizes come to
-    the host, and each expert runs plain GEMMs over its contiguous rows."""
+    device, so the step can sit in a captured graph): one kernel pair over
+    the (row, choice) pairs that streams each chosen expert's weights once.
+    Many rows (prompt portions): the pairs are sorted by expert, the group
+    sizes come to the host, and each expert runs plain GEMMs over its
+    contiguous rows."""
 
     sorted_min_rows = 64
     alpha = 1.702
@@ -221,7 +226,8 @@ class RoutedMoE(nn.Module):
         super().__init__()
         if not (0 < f.top <= f.experts):
             raise ValueError(f"{p}: top must be within 1 .. experts")
-        if f.act not in ("clamp", "silu") or f.score not in ("top", "all"):
+        if f.act not in ("clamp", "silu") or f.score not in (
+                "top", "all", "sigmoid"):
             raise ValueError(f"{p}: unknown expert or router kind")
         if f.groups:
             if f.score != "all" or f.experts % f.groups or \
@@ -258,7 +264,7 @@ class RoutedMoE(nn.Module):
         # in the activation format: products of two bf16 numbers are exact
         # in fp32, so the fp32-output GEMM over bf16 rows IS the fp32 router
         self.w_router = t[p + "router"].to(**dev).contiguous()
-        if f.score == "all" and f.experts % 16:
+        if f.score != "top" and f.experts % 16:
             # the score product is made 16 columns wide at least (zero rows
             # below the experts'); the router reads the first `experts`
             self.w_router = pad_rows(self.w_router, 16)
@@ -276,20 +282,22 @@ class RoutedMoE(nn.Module):
                         "shared.down": (width, f.shared_ff)})
         return out
 
-    def _route(self, idx, wts, logits, dense_rows: int) -> None:
+    def _route(self, idx, wts, logits) -> None:
         """Fill the first `top` columns of idx and wts."""
         f = self.f
-        if f.score == "all":
+        if f.score == "sigmoid":
+            ops.router_sigmoid(idx, wts, logits, f.top, f.route_scale)
+        elif f.score == "all":
             ops.router_select(idx, wts, logits, f.top, f.groups, f.keep,
-                              f.route_scale, dense_rows)
+                              f.route_scale, 0)
         elif idx.shape[1] == f.top:
-            ops.router_topk(idx, wts, logits, f.top, dense_rows)
+            ops.router_topk(idx, wts, logits, f.top, 0)
         else:
             i2 = torch.empty(idx.shape[0], f.top, dtype=idx.dtype,
                              device=idx.device)
             w2 = torch.empty(idx.shape[0], f.top, dtype=wts.dtype,
                              device=idx.device)
-            ops.router_topk(i2, w2, logits, f.top, dense_rows)
+            ops.router_topk(i2, w2, logits, f.top, 0)
             idx[:, :f.top] = i2
             wts[:, :f.top] = w2
 
@@ -310,34 +318,23 @@ class RoutedMoE(nn.Module):
         f = self.f
         T, W = h.shape
         logits = ops.linear_f32(h, self.w_router)[:, :f.experts]
-        # with a shared expert the fold takes one more row per token
-        cols = f.top + (1 if self.shared is not None else 0)
-        idx = torch.empty(T, cols, dtype=torch.int32, device=h.device)
-        wts = torch.empty(T, cols, dtype=torch.float32, device=h.device)
         out = torch.empty_like(h)
         on_host = getattr(meta, "host_ids", None) is not None
-        if on_host and T >= self.sorted_min_rows:
-            self._route(idx, wts, logits, 0)
+        many = on_host and T >= self.sorted_min_rows
+        # with a shared expert the fold of the sorted form takes one more
+        # row per token
+        cols = f.top + (1 if many and self.shared is not None else 0)
+        idx = torch.empty(T, cols, dtype=torch.int32, device=h.device)
+        wts = torch.empty(T, cols, dtype=torch.float32, device=h.device)
+        self._route(idx, wts, logits)
+        if many:
             return self._forward_sorted(out, h, idx, wts)
-        # every expert over every row; idx names rows of the [E*T, W] result
-        self._route(idx, wts, logits, T)
-        E, ff = f.experts, f.ff
-        z = torch.bmm(h.unsqueeze(0).expand(E, T, W),
-                      self.w_gu.transpose(1, 2)).view(E * T, -1)
-        a = torch.empty(E * T, ff, dtype=h.dtype, device=h.device)
-        ops.clamp_glu(a, z[:, :ff], z[:, self.up_col: self.up_col + ff],
-                      None, None, *self.glu)
-        if self.shared is None:
-            y = torch.bmm(a.view(E, T, ff), self.w_down.transpose(1, 2))
-            ops.combine_rows_weighted(out, y.view(E * T, W), idx, wts)
-            return out
-        y = torch.empty((E + 1) * T, W, dtype=h.dtype, device=h.device)
-        torch.bmm(a.view(E, T, ff), self.w_down.transpose(1, 2),
-                  out=y[: E * T].view(E, T, W))
-        self._shared_into(y[E * T:], h)
-        idx[:, f.top] = self._arange(T, h.device) + E * T
-        wts[:, f.top] = 1.0
-        ops.combine_rows_weighted(out, y, idx, wts)
+        extra = None
+        if self.shared is not None:
+            extra = torch.empty_like(h)
+            self._shared_into(extra, h)
+        ops.routed_experts(out, h, idx, wts, f.top, self.w_gu, self.w_down,
+                           *self.glu, f.weigh_input, extra)
         return out
 
     def _arange(self, n: int, device) -> torch.Tensor:
@@ -364,6 +361,11 @@ class RoutedMoE(nn.Module):
         done = torch.empty(T * (top + 1) if shared else T * top, W,
                            dtype=h.dtype, device=h.device)
         a = torch.empty(T * top, ff, dtype=h.dtype, device=h.device)
+        scale = None
+        if f.weigh_input:
+            # the pairs' weights in sorted order; the fold then adds as is
+            scale = wts[:, :top].reshape(-1)[order]
+            wts = torch.ones_like(wts)
         at = 0
         for e in range(E):
             n = counts[e]
@@ -372,7 +374,8 @@ class RoutedMoE(nn.Module):
             z = ops.linear(rows[at: at + n], self.w_gu[e])
             ops.clamp_glu(a[at: at + n], z[:, :ff],
                           z[:, self.up_col: self.up_col + ff], None, None,
-                          *self.glu)
+                          *self.glu,
+                          None if scale is None else scale[at: at + n])
             if n > 64:      # straight into its rows, no copy
                 torch.mm(a[at: at + n], self.w_down[e].t(),
                          out=done[at: at + n])

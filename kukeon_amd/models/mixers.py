@@ -3,7 +3,8 @@ state-space mixer (fixed-size recurrent state per sequence), a latent
 attention mixer (one low-rank row per token in the paged cache), a
 grouped-query attention mixer with chunk-local keys and capped scores, and a
 linear-attention mixer with a fixed decay per head (a state matrix per
-sequence). All take the layer input [T, W] of a packed batch plus the
+sequence), and others with their own memory further down. All take the layer
+input [T, W] of a packed batch plus the
 engine's row maps and return the mixer output [T, W]; all sizes and constants
 are arguments, so any model family can stack them.
 """
@@ -837,3 +838,318 @@ class ParallelMixer(nn.Module):
                               meta, cache_v, buf[:, self.split:],
                               self.right_scale)
         return ops.linear(buf, self.w_o)
+
+
+# ---------------------------------------------------------------------------
+@dataclass
+class DeltaCfg:
+    heads: int
+    kv_heads: int            # query/key heads; heads // kv_heads share one
+    dim: int                 # query/key entries per head
+    vdim: int                # value entries per head
+    conv: int                # taps of the convolutions on q, k and v
+
+
+class DeltaMixer(nn.Module):
+    """Gated delta rule. q, k and v pass a short causal convolution per
+    channel and silu; queries and keys are made unit vectors per head, the
+    queries times dim^(-1/2). Per head, with beta = sigmoid(W_b h) and
+    g = exp(-exp(A_log) softplus(W_a h + dt_bias)),
+
+        S <- g S ;  u = beta (v - S^T k) ;  S <- S + k u^T ;  o = S^T q .
+
+    Each head's o is RMS-normed over its value entries with one weight
+    vector shared by the heads, multiplied by silu(W_g h) and projected out.
+    Carried per sequence (fp32): the last taps-1 projected rows and S^T.
+
+    Tensors (prefix p): q, k [G*dim, W], v, g [H*vdim, W], {q,k,v}.conv
+    [rows, taps], a, b [H, W], A_log, dt_bias [H], norm [vdim],
+    o [W, H*vdim]."""
+
+    def __init__(self, m: DeltaCfg, width: int, eps: float,
+                 t: Dict[str, torch.Tensor], p: str, device, dtype):
+        super().__init__()
+        if m.heads % m.kv_heads:
+            raise ValueError(f"{p}: heads not a multiple of kv_heads")
+        self.m = m
+        self.eps = eps
+        self.col, self.w_in = fuse_rows(
+            [(n, t[p + n]) for n in ("q", "k", "v", "g", "b", "a")], width,
+            dtype, device)
+        f32 = dict(device=device, dtype=torch.float32)
+        # the convolution runs over the first three segments with their
+        # padding columns (zero inputs, zero taps)
+        C = self.col["g"]
+        taps = max(1, m.conv)
+        cw = torch.zeros(taps, C, **f32)
+        for n in ("q", "k", "v"):
+            rows = t[p + n].shape[0]
+            at = self.col[n]
+            if m.conv:
+                w = t[p + n + ".conv"]
+                if tuple(w.shape) != (rows, taps):
+                    raise ValueError(f"{p}{n}.conv: shape {tuple(w.shape)}")
+                cw[:, at: at + rows] = w.to(**f32).t()
+            else:
+                cw[0, at: at + rows] = 1.0
+        self.conv_w = cw.contiguous()
+        self.zero_b = torch.zeros(C, **f32)
+        self.rate = torch.exp(t[p + "A_log"].to(**f32)).contiguous()
+        self.dt_bias = t[p + "dt_bias"].to(**f32).contiguous()
+        self.norm_w = t[p + "norm"].to(**f32).repeat(m.heads).contiguous()
+        self.w_o = nn.Parameter(t[p + "o"].to(device=device, dtype=dtype)
+                                .contiguous(), requires_grad=False)
+
+    @staticmethod
+    def tensor_shapes(m: DeltaCfg, width: int) -> Dict[str, tuple]:
+        Cq, Cv, H = m.kv_heads * m.dim, m.heads * m.vdim, m.heads
+        out = {"q": (Cq, width), "k": (Cq, width), "v": (Cv, width),
+               "g": (Cv, width), "b": (H, width), "a": (H, width),
+               "A_log": (H,), "dt_bias": (H,), "norm": (m.vdim,),
+               "o": (width, Cv)}
+        if m.conv:
+            out.update({"q.conv": (Cq, m.conv), "k.conv": (Cq, m.conv),
+                        "v.conv": (Cv, m.conv)})
+        return out
+
+    def kv_spec(self) -> Optional[LayerKVSpec]:
+        return None
+
+    def state_shape(self):
+        m = self.m
+        return [(self.conv_w.shape[0] - 1, self.conv_w.shape[1]),
+                (m.heads, m.vdim, m.dim)]
+
+    def forward(self, h: torch.Tensor, cache, state, meta,
+                cache_v=None) -> torch.Tensor:
+        m = self.m
+        T = h.shape[0]
+        c = self.col
+        conv_state, S = state
+        taps, C = self.conv_w.shape
+        proj = ops.linear(h, self.w_in)
+        qkv = torch.empty(T, C, dtype=h.dtype, device=h.device)
+        one = meta.max_rows == 1 and T == meta.cu_rows.numel() - 1
+        ops.conv_act(qkv, proj, 0, self.conv_w, self.zero_b, conv_state,
+                     meta.positions, meta.row_seq, meta.cu_rows,
+                     meta.state_slots, 1, one)
+        if not one and taps > 1:
+            ops.conv_tail_update(conv_state, proj, 0, self.zero_b,
+                                 meta.positions, meta.cu_rows,
+                                 meta.state_slots)
+        Cv = m.heads * m.vdim
+        y = torch.empty(T, Cv, dtype=torch.float32, device=h.device)
+        ops.delta_scan(y, qkv, c["q"], c["k"], c["v"], proj, c["b"], c["a"],
+                       self.rate, self.dt_bias, m.dim ** -0.5, S,
+                       meta.positions, meta.cu_rows, meta.state_slots,
+                       m.heads, m.kv_heads, m.dim, m.vdim)
+        o = torch.empty(T, Cv, dtype=h.dtype, device=h.device)
+        ops.head_rmsnorm_gate(o, y, proj[:, c["g"]: c["g"] + Cv],
+                              self.norm_w, m.heads, self.eps, 0)
+        return ops.linear(o, self.w_o)
+
+
+# ---------------------------------------------------------------------------
+@dataclass
+class SinkAttnCfg:
+    heads: int
+    kv_heads: int
+    dim: int                 # query/key entries per head; values = keys
+    scale: float
+    softcap: float = 0.0     # scores become cap tanh(score / cap) (0: off)
+    chunk: int = 0           # keys of the query's own chunk only (0: all)
+    sink: bool = True        # 1 added to the softmax's denominator
+    log_bias: bool = True    # r1_h ln(1 + r2_h (i - j)) off the scores
+
+
+class SinkAttention(nn.Module):
+    """Grouped-query softmax attention whose values are its keys BEFORE
+    their norm. Queries and keys are RMS-normed per head with a weight each;
+    scores are scaled, optionally capped with tanh, lowered by a bias that
+    grows with the logarithm of the distance, and limited to the query's own
+    chunk; the softmax's denominator has a 1 added (a sink of score 0 without
+    a value). The concatenated heads are multiplied by sigmoid of a gate
+    projected from the mixer's input, then projected out.
+
+    One cache row per token and kv head: the key as projected, which is the
+    value. The kernels divide it by its root mean square where they read it
+    for a score, and the key norm's weight is taken over by the queries,
+    (q w_q) . (k / rms(k) w_k) = (q w_q w_k) . k / rms(k).
+
+    Tensors (prefix p): q [H*dim, W], k [G*dim, W], q.norm, k.norm [dim],
+    r1, r2 [H], g [H*dim, W], o [W, H*dim]."""
+
+    def __init__(self, m: SinkAttnCfg, width: int, eps: float,
+                 t: Dict[str, torch.Tensor], p: str, device, dtype):
+        super().__init__()
+        if m.heads % m.kv_heads:
+            raise ValueError(f"{p}: heads not a multiple of kv_heads")
+        self.m = m
+        self.eps = eps
+        self.Cq = m.heads * m.dim
+        self.col, self.w_in = fuse_rows(
+            [("q", t[p + "q"]), ("k", t[p + "k"]), ("g", t[p + "g"])], width,
+            dtype, device)
+        f32 = dict(device=device, dtype=torch.float32)
+        self.qk_norm = (t[p + "q.norm"].to(**f32) *
+                        t[p + "k.norm"].to(**f32)).contiguous()
+        self.r1 = self.r2 = None
+        if m.log_bias:
+            self.r1 = t[p + "r1"].to(**f32).contiguous()
+            self.r2 = t[p + "r2"].to(**f32).contiguous()
+        self.w_o = nn.Parameter(t[p + "o"].to(device=device, dtype=dtype)
+                                .contiguous(), requires_grad=False)
+
+    @staticmethod
+    def tensor_shapes(m: SinkAttnCfg, width: int) -> Dict[str, tuple]:
+        Cq, Ck = m.heads * m.dim, m.kv_heads * m.dim
+        out = {"q": (Cq, width), "k": (Ck, width), "q.norm": (m.dim,),
+               "k.norm": (m.dim,), "g": (Cq, width), "o": (width, Cq)}
+        if m.log_bias:
+            out.update({"r1": (m.heads,), "r2": (m.heads,)})
+        return out
+
+    def kv_spec(self) -> Optional[LayerKVSpec]:
+        return LayerKVSpec(self.m.kv_heads, self.m.dim, 0)
+
+    def state_shape(self):
+        return None
+
+    def forward(self, h: torch.Tensor, cache, state, meta,
+                cache_v=None) -> torch.Tensor:
+        m = self.m
+        T = h.shape[0]
+        c = self.col
+        proj = ops.linear(h, self.w_in)
+        q = torch.empty(T, self.Cq, dtype=h.dtype, device=h.device)
+        ops.head_norm_append(q, cache, proj, c["q"], c["k"], self.qk_norm,
+                             self.eps, meta.positions, meta.row_seq,
+                             meta.block_table)
+        o = torch.empty(T, self.Cq, dtype=h.dtype, device=h.device)
+        if (meta.mode == "prefill" and meta.max_rows >= 16 and
+                meta.qb_seq is not None and
+                ops.masked_tiles_supported(q, m.dim, cache.shape[2])):
+            # prompt portions on the matrix cores
+            ops.masked_attention_tiles(o, q, cache, self.r1, self.r2,
+                                       meta.block_table, meta.seq_lens,
+                                       meta.q_starts, meta.qb_seq,
+                                       meta.qb_start, m.scale, m.softcap,
+                                       m.chunk, m.sink, self.eps)
+        else:
+            ops.masked_attention(o, q, cache, None, None, self.r1, self.r2,
+                                 meta.positions, meta.row_seq,
+                                 meta.block_table, m.heads, m.scale,
+                                 m.softcap, m.chunk, 0, m.sink, self.eps)
+        og = torch.empty_like(o)
+        ops.scaled_gate(og, o, proj[:, c["g"]: c["g"] + self.Cq], 1)
+        return ops.linear(og, self.w_o)
+
+
+# ---------------------------------------------------------------------------
+@dataclass
+class SelectiveCfg:
+    inner: int               # channels
+    state: int               # states per channel
+    dt_rank: int             # inner size of the step's low-rank projection
+    conv: int                # taps of the short convolution
+
+
+class SelectiveMixer(nn.Module):
+    """Selective scan with a decay per (channel, state). The input projection
+    yields [x | z]; x passes a short causal convolution with bias and silu;
+    [dt | B | C] are projected from it, dt <- softplus(W_dt dt + bias) per
+    channel, and with A = -exp(A_log)
+
+        S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n
+        y_c     = sum_n S[c, n] C_n + D_c x_c ,
+
+    then y silu(z) and the output projection. Carried per sequence (fp32):
+    the last taps-1 convolution inputs and S.
+
+    Tensors (prefix p): in [2*inner, W], conv [inner, taps], conv.b [inner],
+    x [dt_rank + 2*state, inner], dt [inner, dt_rank], dt.b [inner],
+    A_log [inner, state], D [inner], o [W, inner]."""
+
+    def __init__(self, m: SelectiveCfg, width: int, eps: float,
+                 t: Dict[str, torch.Tensor], p: str, device, dtype):
+        super().__init__()
+        self.m = m
+        I, N, R = m.inner, m.state, m.dt_rank
+        dev = dict(device=device, dtype=dtype)
+        f32 = dict(device=device, dtype=torch.float32)
+        w_in = t[p + "in"]
+        if w_in.shape[0] != 2 * I:
+            raise ValueError(f"{p}in: rows do not fit the mixer's sizes")
+        self.in_col, self.w_in = fuse_rows(
+            [("x", w_in[:I]), ("z", w_in[I:])], width, dtype, device)
+        taps = max(1, m.conv)
+        if m.conv:
+            cw = t[p + "conv"]
+            if tuple(cw.shape) != (I, taps):
+                raise ValueError(f"{p}conv: shape {tuple(cw.shape)}")
+            self.conv_w = cw.to(**f32).t().contiguous()      # [taps, I]
+            self.conv_b = t[p + "conv.b"].to(**f32).contiguous()
+        else:
+            self.conv_w = torch.ones(1, I, **f32)
+            self.conv_b = torch.zeros(I, **f32)
+        self.zero_b = torch.zeros(I, **f32)
+        w_x = t[p + "x"]
+        # the step's segment is as wide as the (padded) inner size of its
+        # second product: zero rows there, zero columns in W_dt
+        self.rank = -(-R // 16) * 16
+        w1 = torch.zeros(self.rank, I, dtype=w_x.dtype, device=w_x.device)
+        w1[:R] = w_x[:R]
+        self.col, self.w_x = fuse_rows(
+            [("dt", w1), ("B", w_x[R: R + N]), ("C", w_x[R + N:])], I, dtype,
+            device)
+        w2 = torch.zeros(I, self.rank, **dev)
+        w2[:, :R] = t[p + "dt"].to(**dev)
+        self.w_dt = nn.Parameter(w2.contiguous(), requires_grad=False)
+        self.dt_bias = t[p + "dt.b"].to(**f32).contiguous()
+        # a decay is one exp2 of the step times this
+        self.A2 = (-torch.exp(t[p + "A_log"].double()) *
+                   1.4426950408889634).to(**f32).contiguous()
+        self.D = t[p + "D"].to(**f32).contiguous()
+        self.w_o = nn.Parameter(t[p + "o"].to(**dev).contiguous(),
+                                requires_grad=False)
+
+    @staticmethod
+    def tensor_shapes(m: SelectiveCfg, width: int) -> Dict[str, tuple]:
+        I = m.inner
+        out = {"in": (2 * I, width), "x": (m.dt_rank + 2 * m.state, I),
+               "dt": (I, m.dt_rank), "dt.b": (I,), "A_log": (I, m.state),
+               "D": (I,), "o": (width, I)}
+        if m.conv:
+            out.update({"conv": (I, m.conv), "conv.b": (I,)})
+        return out
+
+    def kv_spec(self) -> Optional[LayerKVSpec]:
+        return None
+
+    def state_shape(self):
+        m = self.m
+        return [(self.conv_w.shape[0] - 1, m.inner), (m.inner, m.state)]
+
+    def forward(self, h: torch.Tensor, cache, state, meta,
+                cache_v=None) -> torch.Tensor:
+        m = self.m
+        T = h.shape[0]
+        conv_state, S = state
+        ic, c = self.in_col, self.col
+        proj = ops.linear(h, self.w_in)
+        x = torch.empty(T, m.inner, dtype=h.dtype, device=h.device)
+        one = meta.max_rows == 1 and T == meta.cu_rows.numel() - 1
+        ops.conv_act(x, proj, ic["x"], self.conv_w, self.conv_b, conv_state,
+                     meta.positions, meta.row_seq, meta.cu_rows,
+                     meta.state_slots, 1, one)
+        if not one and self.conv_w.shape[0] > 1:
+            ops.conv_tail_update(conv_state, proj, ic["x"], self.zero_b,
+                                 meta.positions, meta.cu_rows,
+                                 meta.state_slots)
+        dbc = ops.linear(x, self.w_x)
+        dt = ops.linear_f32(dbc[:, c["dt"]: c["dt"] + self.rank], self.w_dt)
+        y = torch.empty(T, m.inner, dtype=h.dtype, device=h.device)
+        ops.selective_scan(y, x, proj[:, ic["z"]: ic["z"] + m.inner], dt,
+                           self.dt_bias, dbc, c["B"], c["C"], self.A2, self.D,
+                           S, meta.positions, meta.cu_rows, meta.state_slots)
+        return ops.linear(y, self.w_o)

@@ -42,6 +42,11 @@ def _bezizen(cfg, device, **kw):
     return BezizenModel(cfg, device=device, **kw)
 
 
+def _noridra(cfg, device, **kw):
+    from kukeon_amd.models.noridra import NoridraModel
+    return NoridraModel(cfg, device=device, **kw)
+
+
 # family -> constructor(cfg, device, **kw)
 FAMILIES: Dict[str, Callable] = {
     "bezizen": _bezizen,
@@ -49,6 +54,7 @@ FAMILIES: Dict[str, Callable] = {
     "llama": _llama,
     "mixtral": _mixtral,
     "lipedra": _lipedra,
+    "noridra": _noridra,
     "rasesun": _rasesun,
 }
 
@@ -58,6 +64,7 @@ ARCHITECTURES: Dict[str, str] = {
     "Rasesun": "rasesun",
     "Dumovik": "dumovik",
     "Bezizen": "bezizen",
+    "Noridra": "noridra",
 }
 
 
@@ -70,6 +77,7 @@ OP_GROUPS: Dict[str, tuple] = {
     "rasesun": ("recur",),
     "dumovik": ("hyb",),
     "bezizen": ("strm",),
+    "noridra": ("delta",),
 }
 
 
@@ -163,13 +171,34 @@ BEZIZEN_PRESETS = {
 }
 
 
+def _noridra_preset(**kw):
+    def make():
+        from kukeon_amd.models.noridra import noridra_bench
+        return noridra_bench(**kw)
+    return make
+
+
+# random-weight Noridra stacks: periods of delta rule, attention, selective
+# scan and delta rule at Llama-3-8B width, and a small one
+NORIDRA_PRESETS = {
+    "noridra-8b-like": _noridra_preset(width=4096, layers=32, heads=32,
+                                       kv_heads=8, ff=14336, vocab=128256,
+                                       name="noridra-8b-like"),
+    "tiny-noridra": _noridra_preset(width=128, layers=4, heads=4, kv_heads=2,
+                                    ff=256, vocab=384, chunk=24, experts=8,
+                                    max_positions=512, name="tiny-noridra"),
+}
+
+
 def preset_names():
     return sorted(list(MODEL_PRESETS) + list(LIPEDRA_PRESETS) +
                   list(RASESUN_PRESETS) + list(DUMOVIK_PRESETS) +
-                  list(BEZIZEN_PRESETS))
+                  list(BEZIZEN_PRESETS) + list(NORIDRA_PRESETS))
 
 
 def preset(name: str):
+    if name in NORIDRA_PRESETS:
+        return NORIDRA_PRESETS[name]()
     if name in BEZIZEN_PRESETS:
         return BEZIZEN_PRESETS[name]()
     if name in DUMOVIK_PRESETS:
@@ -207,5 +236,9 @@ def load_checkpoint(model_dir: str, device, dtype: str = "bf16"):
     if fam == "bezizen":
         from kukeon_amd.models.bezizen import BezizenModel
         return BezizenModel.from_checkpoint(model_dir, device=device,
+                                            dtype=dtype)
+    if fam == "noridra":
+        from kukeon_amd.models.noridra import NoridraModel
+        return NoridraModel.from_checkpoint(model_dir, device=device,
                                             dtype=dtype)
     raise ValueError(f"family {fam} has no checkpoint loader")

@@ -158,33 +158,53 @@ def _strm(t: torch.Tensor):
     return _C_strm
 
 
-def _shared(t: torch.Tensor, first, second):
-    """A kernel that two groups compile from the same source: whichever of
-    the two modules is built serves it (`first` preferred)."""
+_C_delta = None
+_DELTA_IMPORT_ERROR: Exception | None = None
+try:
+    from kukeon_amd import _C_delta  # type: ignore
+except Exception as e:  # pragma: no cover
+    _DELTA_IMPORT_ERROR = e
+
+
+def delta_available() -> bool:
+    return _C_delta is not None
+
+
+def _delta(t: torch.Tensor):
+    """Kernel group of the stacks that norm after the sum (residual norm in
+    runs, input convolution, gated delta rule, selective scan, attention
+    over unnormed keys with a sink, sigmoid routing): native on a GPU tensor
+    (an error if the module is not built), fp32 references on CPU."""
+    global _C_delta, _DELTA_IMPORT_ERROR
     if not t.is_cuda:
         return reference
-    key = (first, second)
-    mod = _SHARED_CHOICE.get(key)
-    if mod is None:
+    if _C_delta is None:
         try:
-            mod = first(t)
-        except RuntimeError:
-            mod = second(t)
-        _SHARED_CHOICE[key] = mod
-    return mod
+            import importlib
+            _C_delta = importlib.import_module("kukeon_amd._C_delta")
+        except Exception as e:
+            _DELTA_IMPORT_ERROR = e
+    if _C_delta is None:
+        raise RuntimeError(
+            "kukeon_amd._C_delta (gfx950 HIP extension) is not built but an "
+            "op was called on a CUDA device. Run `python -m "
+            f"kukeon_amd.ops.build delta` (import error: "
+            f"{_DELTA_IMPORT_ERROR})")
+    return _C_delta
 
 
 _SHARED_CHOICE: dict = {}
 
 
-def _shared3(t: torch.Tensor, first, second, third):
-    """As _shared, for a kernel that three groups compile."""
+def _shared(t: torch.Tensor, *groups):
+    """A kernel that several groups compile from the same source: the first
+    of them whose module is built serves it."""
     if not t.is_cuda:
         return reference
-    key = (first, second, third)
-    mod = _SHARED_CHOICE.get(key)
+    mod = _SHARED_CHOICE.get(groups)
     if mod is None:
-        for get in key:
+        err = None
+        for get in groups:
             try:
                 mod = get(t)
                 break
@@ -192,7 +212,7 @@ def _shared3(t: torch.Tensor, first, second, third):
                 err = e
         if mod is None:
             raise err
-        _SHARED_CHOICE[key] = mod
+        _SHARED_CHOICE[groups] = mod
     return mod
 
 
@@ -489,11 +509,14 @@ def residual_add_rmsnorm(x, a, bias, w, w_offset: float, eps: float,
 
 
 def clamp_glu(out, gate, up, bg, bu, limit: float, alpha: float = 1.702,
-              up_shift: float = 1.0) -> None:
+              up_shift: float = 1.0, row_scale=None) -> None:
+    """`row_scale` [T] multiplies a row's gate and up ahead of everything
+    else."""
     none = torch.empty(0, dtype=torch.float32, device=out.device)
-    _shared3(out, _mix, _hyb, _strm).clamp_glu(
+    _shared(out, _mix, _hyb, _strm, _delta).clamp_glu(
         out, gate, up, bg if bg is not None else none,
-        bu if bu is not None else none, limit, alpha, up_shift)
+        bu if bu is not None else none, limit, alpha, up_shift,
+        row_scale if row_scale is not None else none)
 
 
 def conv_rope_append(q_out, k_cache, v_cache, proj, bias, cw, state, cs,
@@ -594,21 +617,23 @@ def postnorm_residual_rmsnorm(x, y, post_w, w, eps: float, out) -> None:
 
 def conv_act(out, proj, col0: int, cw, bias, state, positions, row_seq,
              cu_rows, state_slots, act: int = 1,
-             shift_state: bool = False) -> None:
+             shift_state: bool = False, skip: bool = False) -> None:
     """Short causal convolution per channel over proj[:, col0:col0+C] with
     carried taps, bias after the sum, then the activation (1: silu, 0:
-    none). With `shift_state` (every sequence brings exactly one row) the
+    none), then, with `skip`, the input itself added. With `shift_state` (every sequence brings exactly one row) the
     same launch shifts the state slots; otherwise conv_tail_update does."""
-    _recur(proj).conv_act(out, proj, col0, cw, bias, state, positions,
-                          row_seq, cu_rows, state_slots, act, shift_state)
+    _shared(proj, _recur, _delta).conv_act(
+        out, proj, col0, cw, bias, state, positions, row_seq, cu_rows,
+        state_slots, act, shift_state, skip)
 
 
 def conv_tail_update(state, proj, col0: int, zero_bias, positions, cu_rows,
                      state_slots) -> None:
     """Shift a portion's last inputs into the convolution state slots."""
     C = state.shape[2]
-    _recur(proj).conv_state_update(state, proj, zero_bias, positions,
-                                   cu_rows, state_slots, col0, 0, 0, C, 0, 0)
+    _shared(proj, _recur, _delta).conv_state_update(
+        state, proj, zero_bias, positions, cu_rows, state_slots, col0, 0, 0,
+        C, 0, 0)
 
 
 def ssm_scan(y, xbc, dt, dt_bias, rate, skip, state, positions, cu_rows,
@@ -650,7 +675,7 @@ def table_moe(out, h, ids, table, w_up, w_down) -> None:
 
 
 def gather_rows(out, inp, row_map) -> None:
-    _shared3(out, _recur, _hyb, _strm).gather_rows(out, inp, row_map)
+    _shared(out, _recur, _hyb, _strm, _delta).gather_rows(out, inp, row_map)
 
 
 def relu_square_(x) -> None:
@@ -734,13 +759,13 @@ def router_topk(idx, wts, logits, top: int, dense_rows: int = 0) -> None:
 
 
 def combine_rows_weighted(out, inp, inv, wts) -> None:
-    _shared(out, _hyb, _strm).combine_rows_weighted(out, inp, inv, wts)
+    _shared(out, _hyb, _strm, _delta).combine_rows_weighted(out, inp, inv, wts)
 
 
 # ---- stream group ----------------------------------------------------------
 def embed_streams(xs, ids, positions, table, pos_table, scale: float) -> None:
     """xs [T, S, W] fp32: every stream = table[id] * scale + pos_table[p]."""
-    _strm(xs).embed_streams(xs, ids, positions, table,
+    _shared(xs, _strm, _delta).embed_streams(xs, ids, positions, table,
                             pos_table if pos_table is not None else _e(table),
                             scale)
 
@@ -784,13 +809,14 @@ def head_rmsnorm_gate(out, y, gate, w, H: int, eps: float, act: int,
                       scale: float = 1.0) -> None:
     """out (a [T, C] view) = y / rms_per_head(y) * w * act(gate) * scale;
     act 0 = silu, 1 = sigmoid."""
-    _strm(out).head_rmsnorm_gate(out, y, gate, w, H, eps, act, scale)
+    _shared(out, _strm, _delta).head_rmsnorm_gate(out, y, gate, w, H, eps,
+                                                  act, scale)
 
 
 def scaled_gate(out, a, gate, act: int, scale: float = 1.0) -> None:
     """out (a [T, C] view) = a * act(gate) * scale; act 0 = silu,
     1 = sigmoid."""
-    _strm(out).scaled_gate(out, a, gate, act, scale)
+    _shared(out, _strm, _delta).scaled_gate(out, a, gate, act, scale)
 
 
 def conv_scale_append(q_out, k_cache, proj, q_col: int, k_col: int, cw, state,
@@ -840,3 +866,109 @@ def router_select(idx, wts, logits, top: int, groups: int, keep: int,
                   scale: float, dense_rows: int = 0) -> None:
     _strm(logits).router_select(idx, wts, logits, top, groups, keep, scale,
                                 dense_rows)
+
+
+# ---- delta group -----------------------------------------------------------
+def routed_experts(out, h, idx, wts, top: int, w_gu, w_down, limit: float,
+                   alpha: float, shift: float, weigh_input: bool = False,
+                   extra=None) -> None:
+    """The chosen experts of a small batch: idx, wts [T, >= top]; the
+    weights multiply the experts' outputs, or their inputs; `extra` [T, W]
+    is added last."""
+    _shared(h, _hyb, _strm, _delta).routed_experts(
+        out, h, idx, wts, top, w_gu, w_down, limit, alpha, shift, weigh_input,
+        extra if extra is not None else _e(h))
+
+
+def postnorm_residual(x, y, alpha: float, scale, w, groups: int, eps: float,
+                      positions) -> None:
+    """x (fp32, in place) <- norm(alpha x + scale y) * w, the RMS norm in
+    `groups` equal runs."""
+    f, i = torch.float32, torch.int32
+    n = lambda dt: torch.empty(0, dtype=dt, device=x.device)
+    _delta(x).postnorm_residual(x, y, alpha, scale, w, groups, eps, positions,
+                                0, n(y.dtype), n(f), n(f), n(f), n(i))
+
+
+def postnorm_residual_conv(x, y, alpha: float, scale, w, groups: int,
+                           eps: float, positions, h, cw, state,
+                           state_slots) -> None:
+    """postnorm_residual, then h = x + conv(x) with the taps before the row
+    from the state slot, which is shifted (every sequence brings one row)."""
+    n = torch.empty(0, dtype=torch.float32, device=x.device)
+    _delta(x).postnorm_residual(x, y, alpha, scale, w, groups, eps, positions,
+                                1, h, n, cw, state, state_slots)
+
+
+def postnorm_residual_norm(x, y, alpha: float, scale, w, groups: int,
+                           eps: float, positions, h, w2) -> None:
+    """postnorm_residual, then h = norm(x) * w2."""
+    n = torch.empty(0, dtype=torch.float32, device=x.device)
+    _delta(x).postnorm_residual(
+        x, y, alpha, scale, w, groups, eps, positions, 2, h, w2, n, n,
+        torch.empty(0, dtype=torch.int32, device=x.device))
+
+
+def delta_scan(y, qkv, q_col: int, k_col: int, v_col: int, ba, b_col: int,
+               a_col: int, rate, dt_bias, q_scale: float, state, positions,
+               cu_rows, state_slots, H: int, G: int, d: int, dv: int) -> None:
+    """Gated delta rule over unit keys and queries; q and k have G heads, v
+    has H."""
+    _delta(qkv).delta_scan(y, qkv, q_col, k_col, v_col, ba, b_col, a_col,
+                           rate, dt_bias, q_scale, state, positions, cu_rows,
+                           state_slots, H, G, d, dv)
+
+
+def selective_scan(out, x, z, dt, dt_bias, bc, b_col: int, c_col: int, A2, D,
+                   state, positions, cu_rows, state_slots) -> None:
+    """Selective scan with a decay per (channel, state), skip and silu gate;
+    A2 = A log2(e)."""
+    _delta(x).selective_scan(out, x, z, dt, dt_bias, bc, b_col, c_col, A2, D,
+                             state, positions, cu_rows, state_slots)
+
+
+def head_norm_append(q_out, k_cache, proj, q_col: int, k_col: int, w,
+                     eps: float, positions, row_seq, block_table) -> None:
+    """Per head q / rms(q) * w into q_out; the key rows go to their page as
+    projected."""
+    _delta(proj).head_norm_append(q_out, k_cache, proj, q_col, k_col, w, eps,
+                                  positions, row_seq, block_table)
+
+
+def masked_attention(out, q, k_cache, v_cache, slopes, r1, r2, positions,
+                     row_seq, block_table, H: int, scale: float,
+                     softcap: float = 0.0, chunk: int = 0, window: int = 0,
+                     sink: bool = False, key_eps: float = -1.0) -> None:
+    """Softmax attention over paged keys with every option of the row kernel:
+    values are the keys when v_cache is None; a linear (slopes) and a
+    logarithmic (r1, r2) distance bias, capped scores, chunk and window,
+    a sink of score 0, keys divided by their root mean square (key_eps >=
+    0)."""
+    none = torch.empty(0, dtype=torch.float32, device=q.device)
+    o = lambda t: t if t is not None else none
+    _delta(q).masked_attention(
+        out, q, k_cache, v_cache if v_cache is not None else _e(q), o(slopes),
+        o(r1), o(r2), positions, row_seq, block_table, H, scale, softcap,
+        chunk, window, sink, key_eps)
+
+
+def masked_tiles_supported(t: torch.Tensor, d: int, BS: int) -> bool:
+    return (t.is_cuda and t.dtype == torch.bfloat16
+            and _delta(t).masked_attention_tiles_supported(d, BS))
+
+
+def masked_attention_tiles(out, q, k_cache, r1, r2, block_table, seq_lens,
+                           q_starts, qb_seq, qb_start, scale: float,
+                           softcap: float, chunk: int, sink: bool,
+                           key_eps: float) -> None:
+    none = torch.empty(0, dtype=torch.float32, device=q.device)
+    _delta(q).masked_attention_tiles(
+        out, q, k_cache, r1 if r1 is not None else none,
+        r2 if r2 is not None else none, block_table, seq_lens, q_starts,
+        qb_seq, qb_start, scale, softcap, chunk, sink, key_eps)
+
+
+def router_sigmoid(idx, wts, logits, top: int, scale: float = 1.0) -> None:
+    """The `top` experts with the largest logits, weights sigmoid(logit)
+    times scale."""
+    _delta(logits).router_sigmoid(idx, wts, logits, top, scale)

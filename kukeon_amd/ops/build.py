@@ -58,6 +58,7 @@ HYB_SOURCES = [
     "prefill_attn.hip",
     "lightning.hip",
     "routed_moe.hip",
+    "routed_experts.hip",
     "latent_attn.hip",
     "recur_elem.hip",
     "table_moe.hip",
@@ -76,9 +77,30 @@ STRM_SOURCES = [
     "chunk_attn.hip",
     "prefill_attn.hip",
     "routed_moe.hip",
+    "routed_experts.hip",
     "glu_clamp.hip",
     "table_moe.hip",
     "bindings_strm.cpp",
+]
+
+#   delta -> kukeon_amd/_C_delta.so (norms after the sum, gated delta rule,
+#                                  selective scan, attention over unnormed
+#                                  keys with a sink, sigmoid-routed experts)
+DELTA_SOURCES = [
+    "post_norm.hip",
+    "conv_act.hip",
+    "short_conv.hip",
+    "delta_scan.hip",
+    "selective_scan.hip",
+    "head_norm.hip",
+    "chunk_attn.hip",
+    "prefill_attn.hip",
+    "stream_mix.hip",
+    "routed_moe.hip",
+    "routed_experts.hip",
+    "glu_clamp.hip",
+    "table_moe.hip",
+    "bindings_delta.cpp",
 ]
 
 SOURCES = [
@@ -114,6 +136,7 @@ GROUPS = {
     "recur": ("_C_recur", RECUR_SOURCES),
     "hyb": ("_C_hyb", HYB_SOURCES),
     "strm": ("_C_strm", STRM_SOURCES),
+    "delta": ("_C_delta", DELTA_SOURCES),
 }
 
 

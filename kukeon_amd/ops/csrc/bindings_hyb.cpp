@@ -14,7 +14,8 @@ void layernorm(torch::Tensor out, torch::Tensor x, torch::Tensor w,
 void gelu_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up);
 void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
                torch::Tensor bg, torch::Tensor bu, double limit, double alpha,
-               double up_shift);
+               double up_shift,
+               torch::Tensor row_scale);
 void qk_norm_append(torch::Tensor q_out, torch::Tensor k_cache,
                     torch::Tensor v_cache, torch::Tensor proj, int64_t q_col,
                     int64_t k_col, int64_t v_col, torch::Tensor wq,
@@ -40,6 +41,10 @@ void gated_rmsnorm(torch::Tensor out, torch::Tensor y, torch::Tensor gate,
                    torch::Tensor w, double eps);
 void router_topk(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
                  int64_t top, int64_t dense_rows);
+void routed_experts(torch::Tensor out, torch::Tensor h, torch::Tensor idx,
+                    torch::Tensor wts, int64_t top, torch::Tensor w_gu,
+                    torch::Tensor w_down, double limit, double alpha,
+                    double shift, bool weigh_input, torch::Tensor extra);
 void combine_rows_weighted(torch::Tensor out, torch::Tensor in,
                            torch::Tensor inv, torch::Tensor wts);
 void head_gate(torch::Tensor out, torch::Tensor o, torch::Tensor gate);
@@ -77,6 +82,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "rmsnorm(y) * w * sigmoid(gate)");
   m.def("router_topk", &kukeon::router_topk,
         "top experts per row and the softmax over their logits");
+  m.def("routed_experts", &kukeon::routed_experts,
+        "the chosen experts of a small batch, by (row, choice) pairs");
   m.def("combine_rows_weighted", &kukeon::combine_rows_weighted,
         "out[t] = sum over k of w[t, k] * in[inv[t, k]]");
   m.def("head_gate", &kukeon::head_gate,

@@ -10,7 +10,8 @@ void residual_add_rmsnorm(torch::Tensor x, torch::Tensor a, torch::Tensor bias,
                           torch::Tensor out);
 void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
                torch::Tensor bg, torch::Tensor bu, double limit, double alpha,
-               double up_shift);
+               double up_shift,
+               torch::Tensor row_scale);
 bool conv_rope_append(torch::Tensor q_out, torch::Tensor k_cache,
                       torch::Tensor v_cache, torch::Tensor proj,
                       torch::Tensor bias, torch::Tensor cw,

@@ -62,11 +62,16 @@ void router_select(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
                    int64_t dense_rows);
 void router_topk(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
                  int64_t top, int64_t dense_rows);
+void routed_experts(torch::Tensor out, torch::Tensor h, torch::Tensor idx,
+                    torch::Tensor wts, int64_t top, torch::Tensor w_gu,
+                    torch::Tensor w_down, double limit, double alpha,
+                    double shift, bool weigh_input, torch::Tensor extra);
 void combine_rows_weighted(torch::Tensor out, torch::Tensor in,
                            torch::Tensor inv, torch::Tensor wts);
 void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
                torch::Tensor bg, torch::Tensor bu, double limit, double alpha,
-               double up_shift);
+               double up_shift,
+               torch::Tensor row_scale);
 void gather_rows(torch::Tensor out, torch::Tensor in, torch::Tensor map);
 }  // namespace kukeon
 
@@ -100,6 +105,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "group-limited choice by softmax scores, normalised weights");
   m.def("router_topk", &kukeon::router_topk,
         "top experts per row and the softmax over their logits");
+  m.def("routed_experts", &kukeon::routed_experts,
+        "the chosen experts of a small batch, by (row, choice) pairs");
   m.def("combine_rows_weighted", &kukeon::combine_rows_weighted,
         "out[t] = sum over k of w[t, k] * in[inv[t, k]]");
   m.def("clamp_glu", &kukeon::clamp_glu,

@@ -4,7 +4,11 @@
 // lo .. p, lo being the first position of p's chunk (0 without chunks). The
 // same kernel serves a sliding window (lo = p - window + 1), a distance bias
 // slope_h (p - j) taken off head h's scores, and caches without value rows,
-// where the values are the keys (window_attention).
+// where the values are the keys (window_attention); and, through
+// masked_attention, a logarithmic distance bias r1_h ln(1 + r2_h (p - j)), keys
+// that are divided by their own root mean square as they are read (the page
+// row stays the value), and a sink, a score of 0 without a value that joins
+// the softmax.
 //
 // qk_norm_append   norms q (and k) of every row, writes q to a dense buffer
 //                  and k, v to the row's page.
@@ -200,6 +204,15 @@ void qk_norm_append(torch::Tensor q_out, torch::Tensor k_cache,
 // ---------------------------------------------------------------------------
 #define CA_HB 4
 
+// what only some designs use: null / 0 / negative switch it off
+struct AttnExtra {
+  const float* slopes;     // [H] linear distance bias
+  const float* r1;         // [H] logarithmic distance bias
+  const float* r2;
+  float key_eps;           // >= 0: keys divided by their root mean square
+  int sink;
+};
+
 // One workgroup per (row, kv head, up to CA_HB of its query heads). Its NW
 // waves (4 for many rows, 16 for few, where the keys are the only source of
 // parallel work) share out the row's key tiles (tile t of 64 keys, counted
@@ -212,7 +225,7 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
     const T* __restrict__ vc, const int* __restrict__ positions,
     const int* __restrict__ row_seq, const int* __restrict__ block_table,
     int max_blocks, int H, int G, int d, int dq, int dv, int BS, float scale,
-    float cap, int chunk, int window, const float* __restrict__ slopes) {
+    float cap, int chunk, int window, AttnExtra ex) {
   extern __shared__ float sm[];
   const int tid = threadIdx.x;
   const int wave = tid / WAVE;
@@ -254,10 +267,13 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
   const int s = row_seq[r];
   int lo = chunk > 0 ? (p / chunk) * chunk : 0;
   if (window > 0) lo = max(lo, p - window + 1);
-  float slope[CA_HB];
+  float slope[CA_HB], lb1[CA_HB], lb2[CA_HB];
 #pragma unroll
-  for (int hb = 0; hb < CA_HB; ++hb)
-    slope[hb] = (slopes && hb < nh) ? slopes[h0 + hb] : 0.f;
+  for (int hb = 0; hb < CA_HB; ++hb) {
+    slope[hb] = (ex.slopes && hb < nh) ? ex.slopes[h0 + hb] : 0.f;
+    lb1[hb] = (ex.r1 && hb < nh) ? ex.r1[h0 + hb] : 0.f;
+    lb2[hb] = (ex.r2 && hb < nh) ? ex.r2[h0 + hb] : 0.f;
+  }
   float m[CA_HB], l[CA_HB], acc[CA_HB][8];
 #pragma unroll
   for (int hb = 0; hb < CA_HB; ++hb) {
@@ -284,10 +300,15 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
       float dot[CA_HB];
 #pragma unroll
       for (int hb = 0; hb < CA_HB; ++hb) dot[hb] = 0.f;
+      float kk = 0.f;
       if (VEC) {
         for (int i = 0; i < d; i += 8) {
           float kv[8];
           ld8(kr + i, kv);
+          if (ex.key_eps >= 0.f) {
+#pragma unroll
+            for (int k = 0; k < 8; ++k) kk = fmaf(kv[k], kv[k], kk);
+          }
 #pragma unroll
           for (int hb = 0; hb < CA_HB; ++hb)
 #pragma unroll
@@ -297,16 +318,21 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
       } else {
         for (int i = 0; i < d; ++i) {
           const float kv = ldf(kr + i);
+          kk = fmaf(kv, kv, kk);
 #pragma unroll
           for (int hb = 0; hb < CA_HB; ++hb)
             dot[hb] = fmaf(kv, sq[hb * dq + i], dot[hb]);
         }
       }
+      const float ks = ex.key_eps >= 0.f
+                           ? scale / sqrtf(kk / (float)d + ex.key_eps)
+                           : scale;
 #pragma unroll
       for (int hb = 0; hb < CA_HB; ++hb) {
-        sc[hb] = dot[hb] * scale;
+        sc[hb] = dot[hb] * ks;
         if (cap > 0.f) sc[hb] = cap * tanhf(sc[hb] / cap);
         sc[hb] -= slope[hb] * (float)(p - j);
+        if (ex.r1) sc[hb] -= lb1[hb] * log1pf(lb2[hb] * (float)(p - j));
       }
     }
 #pragma unroll
@@ -395,10 +421,10 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
   // fold the waves in wave order; a wave without keys has max -inf, weight 0
   for (int i = tid; i < nh * dv; i += blockDim.x) {
     const int hb = i / dv, e = i - hb * dv;
-    float M = -INFINITY;
+    float M = ex.sink ? 0.f : -INFINITY;
     for (int w = 0; w < NW; ++w)
       M = fmaxf(M, sml[(w * CA_HB + hb) * 2]);
-    float num = 0.f, den = 0.f;
+    float num = 0.f, den = ex.sink ? expf(-M) : 0.f;
     for (int w = 0; w < NW; ++w) {
       const float f = expf(sml[(w * CA_HB + hb) * 2] - M);
       num = fmaf(f, smo[(w * CA_HB + hb) * dv + e], num);
@@ -409,13 +435,15 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
 }
 
 // out [T, H*dv], q [T, H*d] contiguous; caches as in qk_norm_append. An
-// empty v_cache means that the values are the keys; slopes [H] fp32 or empty.
-static void masked_attention(torch::Tensor out, torch::Tensor q,
-                             torch::Tensor k_cache, torch::Tensor v_cache,
-                             torch::Tensor slopes, torch::Tensor positions,
-                             torch::Tensor row_seq, torch::Tensor block_table,
-                             int64_t H, double scale, double softcap,
-                             int64_t chunk, int64_t window) {
+// empty v_cache means that the values are the keys; slopes, r1, r2 [H] fp32 or
+// empty.
+void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
+                      torch::Tensor v_cache, torch::Tensor slopes,
+                      torch::Tensor r1, torch::Tensor r2,
+                      torch::Tensor positions, torch::Tensor row_seq,
+                      torch::Tensor block_table, int64_t H, double scale,
+                      double softcap, int64_t chunk, int64_t window,
+                      bool sink, double key_eps) {
   check_act(q, "q");
   if (v_cache.numel() == 0) v_cache = k_cache;
   const bool biased = slopes.numel() > 0;
@@ -423,6 +451,15 @@ static void masked_attention(torch::Tensor out, torch::Tensor q,
     check_f32(slopes, "slopes");
     TORCH_CHECK(slopes.numel() == H);
   }
+  const bool logb = r1.numel() > 0;
+  if (logb) {
+    check_f32(r1, "r1"); check_f32(r2, "r2");
+    TORCH_CHECK(r1.numel() == H && r2.numel() == H);
+  }
+  const AttnExtra ex{biased ? slopes.data_ptr<float>() : nullptr,
+                     logb ? r1.data_ptr<float>() : nullptr,
+                     logb ? r2.data_ptr<float>() : nullptr, (float)key_eps,
+                     (int)sink};
   TORCH_CHECK(window >= 0);
   check_i32(positions, "positions"); check_i32(row_seq, "row_seq");
   check_i32(block_table, "block_table");
@@ -469,7 +506,7 @@ static void masked_attention(torch::Tensor out, torch::Tensor q,
         positions.data_ptr<int>(), row_seq.data_ptr<int>(),                \
         block_table.data_ptr<int>(), (int)block_table.size(1), (int)H, G,  \
         d, dq, dv, BS, (float)scale, (float)softcap, (int)chunk,           \
-        (int)window, biased ? slopes.data_ptr<float>() : nullptr
+        (int)window, ex
   KK_DISPATCH_ACT(q, {
     if (vec) {
       auto kern = chunk_attention_kernel<T, true>;
@@ -503,10 +540,11 @@ void chunk_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                      torch::Tensor v_cache, torch::Tensor positions,
                      torch::Tensor row_seq, torch::Tensor block_table,
                      int64_t H, double scale, double softcap, int64_t chunk) {
-  masked_attention(out, q, k_cache, v_cache,
-                   torch::empty({0}, positions.options().dtype(torch::kFloat32)),
-                   positions, row_seq, block_table, H, scale, softcap, chunk,
-                   0);
+  const auto none =
+      torch::empty({0}, positions.options().dtype(torch::kFloat32));
+  masked_attention(out, q, k_cache, v_cache, none, none, none, positions,
+                   row_seq, block_table, H, scale, softcap, chunk, 0, false,
+                   -1.0);
 }
 
 // Sliding-window attention with a distance bias; an empty v_cache makes the
@@ -516,8 +554,11 @@ void window_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                       torch::Tensor positions, torch::Tensor row_seq,
                       torch::Tensor block_table, int64_t H, double scale,
                       int64_t window) {
-  masked_attention(out, q, k_cache, v_cache, slopes, positions, row_seq,
-                   block_table, H, scale, 0.0, 0, window);
+  const auto none =
+      torch::empty({0}, positions.options().dtype(torch::kFloat32));
+  masked_attention(out, q, k_cache, v_cache, slopes, none, none, positions,
+                   row_seq, block_table, H, scale, 0.0, 0, window, false,
+                   -1.0);
 }
 
 }  // namespace kukeon

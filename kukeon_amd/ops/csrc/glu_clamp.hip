@@ -1,7 +1,8 @@
 // Clamped gated activation for a fused [.. gate .. up ..] projection row:
-//   g = min(gate + bg, limit), u = clamp(up + bu, -limit, limit)
+//   g = min(s gate + bg, limit), u = clamp(s up + bu, -limit, limit)
 //   y = g * sigmoid(alpha * g) * (u + up_shift)
-// The projection biases are added here (in fp32) instead of in the GEMM.
+// The projection biases are added here (in fp32) instead of in the GEMM, and
+// so is an optional factor s per row (the weight of an expert's input).
 // Also the gelu-gated product of a dense gated layer (tanh form of gelu).
 #include "elem.h"
 
@@ -12,13 +13,14 @@ __global__ __launch_bounds__(256) void clamp_glu_kernel(
     T* __restrict__ out, long ldo, const T* __restrict__ gate,
     const T* __restrict__ up, long ldg, const float* __restrict__ bg,
     const float* __restrict__ bu, float limit, float alpha, float up_shift,
-    int F, long total) {
+    int F, long total, const float* __restrict__ row_scale) {
   const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total) return;
   const long r = idx / F;
   const int f = (int)(idx - r * F);
-  float g = ldf(gate + r * ldg + f) + (bg ? bg[f] : 0.f);
-  float u = ldf(up + r * ldg + f) + (bu ? bu[f] : 0.f);
+  const float rs = row_scale ? row_scale[r] : 1.0f;
+  float g = rs * ldf(gate + r * ldg + f) + (bg ? bg[f] : 0.f);
+  float u = rs * ldf(up + r * ldg + f) + (bu ? bu[f] : 0.f);
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
   const float sg = 1.0f / (1.0f + expf(-alpha * g));
@@ -30,7 +32,7 @@ __global__ __launch_bounds__(256) void clamp_glu_vec_kernel(
     T* __restrict__ out, long ldo, const T* __restrict__ gate,
     const T* __restrict__ up, long ldg, const float* __restrict__ bg,
     const float* __restrict__ bu, float limit, float alpha, float up_shift,
-    int F8, long total8) {
+    int F8, long total8, const float* __restrict__ row_scale) {
   const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total8) return;
   const long r = idx / F8;
@@ -38,6 +40,11 @@ __global__ __launch_bounds__(256) void clamp_glu_vec_kernel(
   float g[8], u[8], y[8];
   ld8(gate + r * ldg + f, g);
   ld8(up + r * ldg + f, u);
+  if (row_scale) {
+    const float rs = row_scale[r];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) { g[k] *= rs; u[k] *= rs; }
+  }
   if (bg) {
     float t[8], s[8];
     ld8(bg + f, t);
@@ -55,10 +62,11 @@ __global__ __launch_bounds__(256) void clamp_glu_vec_kernel(
 }
 
 // out [T,F] view (stride(1)==1); gate, up [T,F] views into one projection
-// buffer sharing a row stride; bg, bu [F] fp32 or empty.
+// buffer sharing a row stride; bg, bu [F] fp32 or empty; row_scale [T] fp32 or
+// empty.
 void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
                torch::Tensor bg, torch::Tensor bu, double limit, double alpha,
-               double up_shift) {
+               double up_shift, torch::Tensor row_scale) {
   check_act(out, "out");
   TORCH_CHECK(gate.scalar_type() == out.scalar_type() &&
               up.scalar_type() == out.scalar_type());
@@ -74,6 +82,12 @@ void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
     check_f32(bg, "bg");
     check_f32(bu, "bu");
     TORCH_CHECK(bg.numel() == F && bu.numel() == F);
+  }
+  const float* rsp = nullptr;
+  if (row_scale.numel() > 0) {
+    check_f32(row_scale, "row_scale");
+    TORCH_CHECK(row_scale.numel() == rows);
+    rsp = row_scale.data_ptr<float>();
   }
   const long total = rows * F;
   if (total == 0) return;
@@ -91,7 +105,7 @@ void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
           reinterpret_cast<const T*>(up.data_ptr()), gate.stride(0),
           hb ? bg.data_ptr<float>() : nullptr,
           hb ? bu.data_ptr<float>() : nullptr, (float)limit, (float)alpha,
-          (float)up_shift, F / 8, total8);
+          (float)up_shift, F / 8, total8, rsp);
     });
     HIP_CHECK_KERNEL();
     return;
@@ -104,7 +118,7 @@ void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
         reinterpret_cast<const T*>(up.data_ptr()), gate.stride(0),
         hb ? bg.data_ptr<float>() : nullptr,
         hb ? bu.data_ptr<float>() : nullptr, (float)limit, (float)alpha,
-        (float)up_shift, F, total);
+        (float)up_shift, F, total, rsp);
   });
   HIP_CHECK_KERNEL();
 }

@@ -129,8 +129,12 @@ DEV_INLINE unsigned int cvt_pk_bf16(float lo, float hi) {
 // so that they keep fp32-grade accuracy. EXT also serves a sliding window
 // (keys from q - window + 1 on) and a distance bias slope_h (q - k) taken off
 // head h's scores; with the key cache passed as the value cache too, the
-// values are the keys.
-template <int BS, bool FP8, bool EXT>
+// values are the keys. EXT == 2 takes besides a logarithmic distance bias
+// r1_h ln(1 + r2_h (q - k)) (a wave's 63 distances of a tile are one logarithm
+// per lane, handed over through LDS), keys divided by their own root mean
+// square (formed while the tile is staged), and a sink: the softmax starts from
+// a score of 0 that has no value.
+template <int BS, bool FP8, int EXT>
 __global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
     unsigned short* __restrict__ out,       // [T, Hq*D]
     const unsigned short* __restrict__ q,   // [T, q_stride] fused qkv rows
@@ -143,12 +147,15 @@ __global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
     const int* __restrict__ qb_start,       // [nqb] local q offset
     long q_stride, long q_offset, int Hq, int Hk, int max_blocks,
     int out_stride, float scale, float cap, int chunk, int window,
-    const float* __restrict__ slopes) {
+    const float* __restrict__ slopes, const float* __restrict__ r1,
+    const float* __restrict__ r2, float key_eps, int sink) {
   constexpr int D = 128;
   constexpr int KVT = 32;
   // 16-B aligned: staged via uint4 stores (guide G17)
   __shared__ __align__(16) unsigned short kbuf[KVT * D];   // XOR-swizzled K
   __shared__ __align__(16) unsigned short vtbuf[D * KVT];  // V^T tile
+  __shared__ __align__(16) float kscale[EXT == 2 ? KVT : 4];   // EXT == 2
+  __shared__ float dbias[EXT == 2 ? 4 : 1][WAVE];
 
   const int s = qb_seq[blockIdx.x];
   const int qb0 = qb_start[blockIdx.x];
@@ -178,6 +185,8 @@ __global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
     tile_lo = max(tile_lo, abs_start + qb0 - window + 1);
   }
   const float slope = (EXT && slopes) ? slopes[head] : 0.f;
+  const float lb1 = (EXT == 2 && r1) ? r1[head] : 0.f;
+  const float lb2 = (EXT == 2 && r1) ? r2[head] : 0.f;
 
   // ---- load Q fragments (B-operand: col=q, k=d chunks) ----
   unsigned int qfrag[8][4];
@@ -193,6 +202,7 @@ __global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
   }
 
   float m = -INFINITY, l_acc = 0.f;
+  if (EXT == 2 && sink) { m = 0.f; l_acc = 1.f; }
   f32x16_t oacc[4] = {{}, {}, {}, {}};
 
   const int kv_limit = min(ctx, abs_start + qb0 + qn);
@@ -212,6 +222,7 @@ __global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
       const int pblk = block_table[(long)s * max_blocks + bidx];
       const long koff = (((long)pblk * Hk + hk) * BS + (kvpos % BS)) * D;
       const int swz = (tok & 15) << 4;
+      float kk = 0.f;
 #pragma unroll
       for (int c = 0; c < 2; ++c) {
         uint4 v;
@@ -227,6 +238,21 @@ __global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
         const int byte = tok * 256 + (((d0 + c * 8) * 2) ^ swz);
         *reinterpret_cast<uint4*>(
             reinterpret_cast<char*>(kbuf) + byte) = v;
+        if (EXT == 2) {
+          const bf16x8 kv{v};
+#pragma unroll
+          for (int j = 0; j < 8; ++j) kk = fmaf(kv.f(j), kv.f(j), kk);
+        }
+      }
+      if (EXT == 2) {
+        // the row's 8 threads are neighbours
+        kk += __shfl_xor(kk, 1, WAVE);
+        kk += __shfl_xor(kk, 2, WAVE);
+        kk += __shfl_xor(kk, 4, WAVE);
+        if ((threadIdx.x & 7) == 0)
+          kscale[tok] = key_eps >= 0.f
+                            ? scale / sqrtf(kk / (float)D + key_eps)
+                            : scale;
       }
       // V: thread covers (kv pair = tid/16, d0 = (tid%16)*8), transpose
       const int kp = threadIdx.x >> 4;          // 0..15 -> kv = 2*kp
@@ -291,15 +317,32 @@ __global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
     // ---- online softmax over this lane's 16 kv rows ----
     float sv[16];
     float tmax = -INFINITY;
+    if (EXT == 2) {
+      // entry i: the bias at distance (first query) - (last key) + i
+      const int dist = abs_start + qb0 - kvbase - 31 + lane;
+      dbias[wid][lane] = lb1 * __logf(1.0f + lb2 * (float)max(dist, 0));
+      __builtin_amdgcn_wave_barrier();   // wave-private, in order
+    }
+    const float cap2 = 2.0f / cap;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int kvrow = (r & 3) + 8 * (r >> 2) + 4 * hi;
       const int kvpos = kvbase + kvrow;
       const bool valid = (kvpos <= q_abs) && (kvpos < ctx) &&
                          (!EXT || kvpos >= q_lo);
-      float sc = sacc[r] * scale;
-      if (EXT && cap > 0.f) sc = cap * tanhf(sc / cap);
-      if (EXT) sc -= slope * (float)(q_abs - kvpos);
+      float sc;
+      if (EXT == 2) {
+        sc = sacc[r] * kscale[kvrow];
+        // cap tanh(sc / cap); the exponential's overflow gives exactly cap
+        if (cap > 0.f)
+          sc = cap - 2.0f * cap *
+                         __builtin_amdgcn_rcpf(1.0f + __expf(sc * cap2));
+        sc -= dbias[wid][qcol - kvrow + 31];
+      } else {
+        sc = sacc[r] * scale;
+        if (EXT && cap > 0.f) sc = cap * tanhf(sc / cap);
+        if (EXT) sc -= slope * (float)(q_abs - kvpos);
+      }
       sv[r] = valid ? sc : -INFINITY;
       tmax = fmaxf(tmax, sv[r]);
     }
@@ -419,14 +462,14 @@ void prefill_attention(torch::Tensor out, torch::Tensor q,
   dim3 grid(nqb, Hk, (G + 3) / 4);
   const bool fp8 = k_cache.scalar_type() == torch::kUInt8;
 #define PF_LAUNCH(FP8_)                                                      \
-  prefill_attn_kernel<16, FP8_, false><<<grid, 256, 0, stream>>>(            \
+  prefill_attn_kernel<16, FP8_, 0><<<grid, 256, 0, stream>>>(            \
       reinterpret_cast<unsigned short*>(out.data_ptr()),                     \
       reinterpret_cast<const unsigned short*>(q.data_ptr()),                 \
       k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr<int>(),   \
       seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),                    \
       qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0),         \
       q_offset, Hq, Hk, (int)block_table.size(1), (int)out.stride(0),        \
-      (float)scale, 0.f, 0, 0, nullptr)
+      (float)scale, 0.f, 0, 0, nullptr, nullptr, nullptr, -1.f, 0)
   if (fp8) { PF_LAUNCH(true); } else { PF_LAUNCH(false); }
 #undef PF_LAUNCH
   HIP_CHECK_KERNEL();
@@ -472,14 +515,14 @@ void chunk_attention_tiles(torch::Tensor out, torch::Tensor q,
   const int G = Hq / Hk;
   auto stream = c10::hip::getCurrentHIPStream().stream();
   dim3 grid(nqb, Hk, (G + 3) / 4);
-  prefill_attn_kernel<16, false, true><<<grid, 256, 0, stream>>>(
+  prefill_attn_kernel<16, false, 1><<<grid, 256, 0, stream>>>(
       reinterpret_cast<unsigned short*>(out.data_ptr()),
       reinterpret_cast<const unsigned short*>(q.data_ptr()),
       k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr<int>(),
       seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),
       qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0), 0L, Hq,
       Hk, (int)block_table.size(1), (int)out.stride(0), (float)scale,
-      (float)softcap, (int)chunk, 0, nullptr);
+      (float)softcap, (int)chunk, 0, nullptr, nullptr, nullptr, -1.f, 0);
   HIP_CHECK_KERNEL();
 }
 
@@ -525,14 +568,68 @@ void window_attention_tiles(torch::Tensor out, torch::Tensor q,
   const int G = Hq / Hk;
   auto stream = c10::hip::getCurrentHIPStream().stream();
   dim3 grid(nqb, Hk, (G + 3) / 4);
-  prefill_attn_kernel<16, false, true><<<grid, 256, 0, stream>>>(
+  prefill_attn_kernel<16, false, 1><<<grid, 256, 0, stream>>>(
       reinterpret_cast<unsigned short*>(out.data_ptr()),
       reinterpret_cast<const unsigned short*>(q.data_ptr()),
       k_cache.data_ptr(), k_cache.data_ptr(), block_table.data_ptr<int>(),
       seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),
       qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0), 0L, Hq,
       Hk, (int)block_table.size(1), (int)out.stride(0), (float)scale, 0.f, 0,
-      (int)window, biased ? slopes.data_ptr<float>() : nullptr);
+      (int)window, biased ? slopes.data_ptr<float>() : nullptr, nullptr,
+      nullptr, -1.f, 0);
+  HIP_CHECK_KERNEL();
+}
+
+// Prompt portions of chunk-local attention over key-only pages (the values are
+// the keys) with capped scores, a logarithmic distance bias, keys divided by
+// their root mean square as they are read (key_eps >= 0) and a sink: out, q
+// [T, H*128] contiguous, k_cache [blocks, G, 16, 128], r1, r2 [H] fp32 or
+// empty.
+void masked_attention_tiles(torch::Tensor out, torch::Tensor q,
+                            torch::Tensor k_cache, torch::Tensor r1,
+                            torch::Tensor r2, torch::Tensor block_table,
+                            torch::Tensor seq_lens, torch::Tensor q_starts,
+                            torch::Tensor qb_seq, torch::Tensor qb_start,
+                            double scale, double softcap, int64_t chunk,
+                            bool sink, double key_eps) {
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous());
+  const int Hk = (int)k_cache.size(1);
+  TORCH_CHECK(window_attention_tiles_supported(k_cache.size(3),
+                                               k_cache.size(2)));
+  TORCH_CHECK(q.scalar_type() == torch::kBFloat16 &&
+              out.scalar_type() == torch::kBFloat16 &&
+              k_cache.scalar_type() == torch::kBFloat16);
+  TORCH_CHECK(q.dim() == 2 && q.is_contiguous() && out.dim() == 2 &&
+              out.is_contiguous() && out.size(0) == q.size(0) &&
+              out.size(1) == q.size(1) && q.size(1) % 128 == 0);
+  const int Hq = (int)(q.size(1) / 128);
+  TORCH_CHECK(Hq % Hk == 0 && chunk >= 0);
+  const bool logb = r1.numel() > 0;
+  if (logb)
+    for (const auto& t : {r1, r2})
+      TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 &&
+                  t.is_contiguous() && t.numel() == Hq);
+  TORCH_CHECK(q_starts.dim() == 2 && q_starts.size(1) == 2);
+  TORCH_CHECK(qb_seq.scalar_type() == torch::kInt32 &&
+              qb_start.scalar_type() == torch::kInt32 &&
+              seq_lens.scalar_type() == torch::kInt32 &&
+              block_table.scalar_type() == torch::kInt32 &&
+              q_starts.scalar_type() == torch::kInt32);
+  const int nqb = (int)qb_seq.size(0);
+  if (nqb == 0) return;
+  const int G = Hq / Hk;
+  auto stream = c10::hip::getCurrentHIPStream().stream();
+  dim3 grid(nqb, Hk, (G + 3) / 4);
+  prefill_attn_kernel<16, false, 2><<<grid, 256, 0, stream>>>(
+      reinterpret_cast<unsigned short*>(out.data_ptr()),
+      reinterpret_cast<const unsigned short*>(q.data_ptr()),
+      k_cache.data_ptr(), k_cache.data_ptr(), block_table.data_ptr<int>(),
+      seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),
+      qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0), 0L, Hq,
+      Hk, (int)block_table.size(1), (int)out.stride(0), (float)scale,
+      (float)softcap, (int)chunk, 0, nullptr,
+      logb ? r1.data_ptr<float>() : nullptr,
+      logb ? r2.data_ptr<float>() : nullptr, (float)key_eps, (int)sink);
   HIP_CHECK_KERNEL();
 }
 

@@ -5,6 +5,8 @@
 //                          equal runs of neighbours of which only the best
 //                          few (by their largest score) can be chosen; the
 //                          chosen scores are divided by their sum and scaled
+//   router_sigmoid         scores = sigmoid of every logit by itself; the `top`
+//                          largest, as they are, times a scale
 //   combine_rows_weighted  out[t] = sum_k w[t, k] * in[inv[t, k]], the k-th
 //                          term added k-th, fp32 sums
 // The expert GEMMs themselves are vendor GEMMs over gathered rows.
@@ -169,6 +171,58 @@ void router_select(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
       (long)wts.stride(0), logits.data_ptr<float>(), (long)logits.stride(0),
       rows, E, (int)top, (int)groups, (int)keep, (float)scale,
       (long)dense_rows);
+  HIP_CHECK_KERNEL();
+}
+
+// One thread per row; a sigmoid keeps the order of the logits.
+__global__ __launch_bounds__(64) void router_sigmoid_kernel(
+    int* __restrict__ idx, float* __restrict__ wts, long ldi, long ldw,
+    const float* __restrict__ logits, long ldz, long rows, int E, int top,
+    float scale) {
+  const long t = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (t >= rows) return;
+  const float* z = logits + t * ldz;
+  float pv = INFINITY;
+  int pe = -1;
+  for (int k = 0; k < top; ++k) {
+    float bv = -INFINITY;
+    int be = -1;
+    for (int e = 0; e < E; ++e) {
+      float v = z[e];
+      v = v == v ? v : -INFINITY;
+      const bool below = v < pv || (v == pv && e > pe);
+      const bool better = be < 0 || v > bv;
+      if (below && better) { bv = v; be = e; }
+    }
+    pv = bv;
+    pe = be;
+    wts[t * ldw + k] = scale / (1.0f + expf(-bv));
+    idx[t * ldi + k] = be;
+  }
+}
+
+// idx [T, >= top] int32, wts [T, >= top] fp32, logits [T, E] fp32 (row strides
+// free).
+void router_sigmoid(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
+                    int64_t top, double scale) {
+  TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == torch::kFloat32 &&
+              logits.dim() == 2 && logits.stride(1) == 1,
+              "logits must be fp32 rows");
+  TORCH_CHECK(idx.is_cuda() && idx.scalar_type() == torch::kInt32 &&
+              wts.is_cuda() && wts.scalar_type() == torch::kFloat32);
+  TORCH_CHECK(idx.dim() == 2 && wts.dim() == 2);
+  const long rows = logits.size(0);
+  const int E = (int)logits.size(1);
+  TORCH_CHECK(top >= 1 && top <= E);
+  TORCH_CHECK(idx.size(0) == rows && wts.size(0) == rows &&
+              idx.size(1) >= top && wts.size(1) >= top &&
+              idx.stride(1) == 1 && wts.stride(1) == 1);
+  if (rows == 0) return;
+  auto stream = c10::hip::getCurrentHIPStream().stream();
+  router_sigmoid_kernel<<<dim3((unsigned)((rows + 63) / 64)), 64, 0, stream>>>(
+      idx.data_ptr<int>(), wts.data_ptr<float>(), (long)idx.stride(0),
+      (long)wts.stride(0), logits.data_ptr<float>(), (long)logits.stride(0),
+      rows, E, (int)top, (float)scale);
   HIP_CHECK_KERNEL();
 }
 

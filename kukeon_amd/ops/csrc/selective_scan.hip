@@ -1,0 +1,235 @@
+// Selective scan with a decay per (channel, state) pair, the recurrent form:
+//
+//   dt_t = softplus(dt_raw_t + dt_bias)                       per channel
+//   S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n
+//   y_c  = sum_n S[c, n] C_n + D_c x_c ;   out = y * silu(z)
+//
+// The channels are independent; B and C are shared by all of them. LN lanes
+// own a channel's state row in interleaved pieces of four (state = (4 i +
+// lane) 4 + j), in registers for the whole portion, next to the channel's row
+// of A (given as A log2(e), so that a decay is one exp2). B and C of TT tokens
+// are staged in LDS at a time, padded with zeros; a thread fetches its
+// channel's x, dt and z of several tokens ahead of the recurrence. The slot
+// ([inner, state]) is read once at the start of the portion (zeros at position
+// 0, whatever the slot held) and written once at its end. Tokens are visited
+// in order, so a position's result does not depend on how the sequence was
+// cut. Everything is fp32.
+#include "elem.h"
+
+namespace kukeon {
+
+#define SS_TT 32
+#define SS_PF 8                 // tokens fetched ahead
+
+template <int CTRL>
+DEV_INLINE float ss_dpp_add(float v) {
+  const int m = __builtin_amdgcn_update_dpp(
+      0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true);
+  return v + __builtin_bit_cast(float, m);
+}
+template <int LN>
+DEV_INLINE float ss_lanes_sum(float v) {
+  if (LN > 1) v = ss_dpp_add<0xB1>(v);
+  if (LN > 2) v = ss_dpp_add<0x4E>(v);
+  if (LN > 4) v = ss_dpp_add<0x141>(v);
+  if (LN > 8) v = ss_dpp_add<0x140>(v);
+  return v;
+}
+
+template <typename T, int LN, int NR>
+__global__ __launch_bounds__(256) void selective_scan_kernel(
+    T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ z,
+    long ldz, const float* __restrict__ dt, long lddt,
+    const float* __restrict__ dt_bias,
+    const T* __restrict__ bc, long ldbc, long b_col, long c_col,
+    const float* __restrict__ A2, const float* __restrict__ D,
+    float* __restrict__ state, const int* __restrict__ positions,
+    const int* __restrict__ cu_rows, const int* __restrict__ state_slots,
+    int I, int N) {
+  constexpr int NP = LN * NR;
+  constexpr int NC = 256 / LN;
+  __shared__ __align__(16) float sB[SS_TT * NP];
+  __shared__ __align__(16) float sC[SS_TT * NP];
+  const int s = blockIdx.x;
+  const long row0 = cu_rows[s];
+  const int n = cu_rows[s + 1] - (int)row0;
+  if (n <= 0) return;
+  const int p0 = positions[row0];
+  const int tid = threadIdx.x;
+  const int l = tid % LN;
+  const int c = blockIdx.y * NC + tid / LN;
+  const bool live = c < I;
+  const int cc = live ? c : 0;
+  if (p0 < 0) {                          // inactive sequence: zeros out
+    if (live && l == 0)
+      for (int t = 0; t < n; ++t) stf(out + (row0 + t) * (long)I + c, 0.f);
+    return;
+  }
+  const float bias = dt_bias[cc], skip = D[cc];
+  float* st = state + ((long)state_slots[s] * I + cc) * (long)N;
+  const float* ar = A2 + (long)cc * N;
+  const bool vec4 = (N & 3) == 0;
+  float S[NR], A[NR];
+#pragma unroll
+  for (int i = 0; i < NR / 4; ++i) {
+    const int nn = (i * LN + l) * 4;
+    float4 sv = float4{0.f, 0.f, 0.f, 0.f}, av = sv;
+    if (vec4) {
+      if (nn < N) {
+        av = *reinterpret_cast<const float4*>(ar + nn);
+        if (p0 > 0) sv = *reinterpret_cast<const float4*>(st + nn);
+      }
+    } else {
+      float* sp = &sv.x;
+      float* ap = &av.x;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (nn + j < N) {
+          ap[j] = ar[nn + j];
+          if (p0 > 0) sp[j] = st[nn + j];
+        }
+    }
+    S[4 * i] = sv.x; S[4 * i + 1] = sv.y; S[4 * i + 2] = sv.z; S[4 * i + 3] = sv.w;
+    A[4 * i] = av.x; A[4 * i + 1] = av.y; A[4 * i + 2] = av.z; A[4 * i + 3] = av.w;
+  }
+  for (int t0 = 0; t0 < n; t0 += SS_TT) {
+    const int nt = min(SS_TT, n - t0);
+    __syncthreads();
+    for (int i = tid; i < nt * NP; i += 256) {
+      const int t = i / NP, nn = i - t * NP;
+      const T* row = bc + (row0 + t0 + t) * ldbc + nn;
+      sB[i] = nn < N ? ldf(row + b_col) : 0.f;
+      sC[i] = nn < N ? ldf(row + c_col) : 0.f;
+    }
+    __syncthreads();
+    for (int t1 = 0; t1 < nt; t1 += SS_PF) {
+      const int np = min(SS_PF, nt - t1);
+      const long r1 = row0 + t0 + t1;
+      float px[SS_PF], pd[SS_PF], pz[SS_PF];
+#pragma unroll
+      for (int k = 0; k < SS_PF; ++k) {
+        px[k] = 0.f; pd[k] = 0.f; pz[k] = 0.f;
+        if (k < np) {
+          px[k] = ldf(x + (r1 + k) * (long)I + cc);
+          pd[k] = dt[(r1 + k) * lddt + cc];
+          pz[k] = ldf(z + (r1 + k) * ldz + cc);
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < SS_PF; ++k) {
+        if (k >= np) break;
+        const float a = pd[k] + bias;
+        const float step = a > 20.f ? a : log1pf(expf(a));
+        const float dx = step * px[k];
+        const float4* bt =
+            reinterpret_cast<const float4*>(sB + (t1 + k) * NP) + l;
+        const float4* ct =
+            reinterpret_cast<const float4*>(sC + (t1 + k) * NP) + l;
+        float acc[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < NR / 4; ++i) {
+          const float4 b4 = bt[i * LN];
+          const float4 c4 = ct[i * LN];
+          const float bb[4] = {b4.x, b4.y, b4.z, b4.w};
+          const float c_[4] = {c4.x, c4.y, c4.z, c4.w};
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const int m = 4 * i + j;
+            S[m] = fmaf(__builtin_amdgcn_exp2f(step * A[m]), S[m], dx * bb[j]);
+            acc[j] = fmaf(S[m], c_[j], acc[j]);
+          }
+        }
+        float yv = ss_lanes_sum<LN>((acc[0] + acc[1]) + (acc[2] + acc[3]));
+        if (live && l == 0) {
+          yv = fmaf(skip, px[k], yv);
+          const float g = pz[k] / (1.0f + expf(-pz[k]));
+          stf(out + (r1 + k) * (long)I + c, yv * g);
+        }
+      }
+    }
+  }
+  if (live) {
+#pragma unroll
+    for (int i = 0; i < NR / 4; ++i) {
+      const int nn = (i * LN + l) * 4;
+      if (vec4) {
+        if (nn < N)
+          *reinterpret_cast<float4*>(st + nn) =
+              float4{S[4 * i], S[4 * i + 1], S[4 * i + 2], S[4 * i + 3]};
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (nn + j < N) st[nn + j] = S[4 * i + j];
+      }
+    }
+  }
+}
+
+// out, x [T, I] contiguous; z [T, I] view (stride(1) == 1); dt [T, I] fp32
+// (stride(1) == 1), before bias and softplus; bc [T, ld]: N columns of B from
+// b_col and of C from c_col; A2 [I, N] = A log2(e), dt_bias, D [I] fp32; state
+// [slots, I, N] fp32.
+void selective_scan(torch::Tensor out, torch::Tensor x, torch::Tensor z,
+                    torch::Tensor dt, torch::Tensor dt_bias, torch::Tensor bc,
+                    int64_t b_col, int64_t c_col, torch::Tensor A2,
+                    torch::Tensor D, torch::Tensor state,
+                    torch::Tensor positions, torch::Tensor cu_rows,
+                    torch::Tensor state_slots) {
+  check_act(out, "out"); check_act(x, "x"); check_act(z, "z");
+  check_act(bc, "bc");
+  check_f32(dt_bias, "dt_bias"); check_f32(A2, "A2"); check_f32(D, "D");
+  check_f32(state, "state");
+  check_i32(positions, "positions"); check_i32(cu_rows, "cu_rows");
+  check_i32(state_slots, "state_slots");
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && out.is_contiguous() &&
+              out.sizes() == x.sizes() && out.scalar_type() == x.scalar_type());
+  const long rows = x.size(0), I = x.size(1);
+  TORCH_CHECK(z.dim() == 2 && z.size(0) == rows && z.size(1) == I &&
+              z.stride(1) == 1 && z.scalar_type() == x.scalar_type());
+  TORCH_CHECK(dt.is_cuda() && dt.scalar_type() == torch::kFloat32 &&
+              dt.dim() == 2 && dt.size(0) == rows && dt.size(1) == I &&
+              dt.stride(1) == 1, "dt must be fp32 rows");
+  TORCH_CHECK(A2.dim() == 2 && A2.size(0) == I);
+  const long N = A2.size(1);
+  TORCH_CHECK(bc.dim() == 2 && bc.size(0) == rows && bc.stride(1) == 1 &&
+              bc.scalar_type() == x.scalar_type() && b_col >= 0 &&
+              b_col + N <= bc.size(1) && c_col >= 0 && c_col + N <= bc.size(1));
+  TORCH_CHECK(dt_bias.numel() == I && D.numel() == I);
+  TORCH_CHECK(state.dim() == 3 && state.size(1) == I && state.size(2) == N);
+  TORCH_CHECK(positions.numel() == rows);
+  const long nseq = cu_rows.numel() - 1;
+  TORCH_CHECK(nseq >= 0 && state_slots.numel() >= nseq);
+  if (rows == 0 || nseq == 0) return;
+  TORCH_CHECK(N >= 1 && N <= 128, "selective_scan: 1 to 128 states per channel");
+  auto stream = c10::hip::getCurrentHIPStream().stream();
+#define KK_LAUNCH(LN_, NR_)                                                   \
+  {                                                                           \
+    constexpr long NC_ = 256 / LN_;                                           \
+    dim3 grid((unsigned)nseq, (unsigned)((I + NC_ - 1) / NC_));               \
+    selective_scan_kernel<T, LN_, NR_><<<grid, 256, 0, stream>>>(             \
+        reinterpret_cast<T*>(out.data_ptr()),                                 \
+        reinterpret_cast<const T*>(x.data_ptr()),                             \
+        reinterpret_cast<const T*>(z.data_ptr()), (long)z.stride(0),          \
+        dt.data_ptr<float>(), (long)dt.stride(0), dt_bias.data_ptr<float>(),  \
+        reinterpret_cast<const T*>(bc.data_ptr()), (long)bc.stride(0),        \
+        (long)b_col, (long)c_col, A2.data_ptr<float>(), D.data_ptr<float>(),  \
+        state.data_ptr<float>(), positions.data_ptr<int>(),                   \
+        cu_rows.data_ptr<int>(), state_slots.data_ptr<int>(), (int)I,         \
+        (int)N);                                                              \
+  }
+  // one token per sequence, or too few channels to fill the device: spread a
+  // channel's states over lanes; otherwise keep them in one or two threads
+  const bool spread = rows == nseq || nseq * I < 128 * 1024;
+  KK_DISPATCH_ACT(x, {
+    if (N <= 4) KK_LAUNCH(1, 4)
+    else if (N <= 8) { if (spread) KK_LAUNCH(2, 4) else KK_LAUNCH(1, 8) }
+    else if (N <= 16) { if (spread) KK_LAUNCH(4, 4) else KK_LAUNCH(1, 16) }
+    else if (N <= 32) { if (spread) KK_LAUNCH(8, 4) else KK_LAUNCH(2, 16) }
+    else if (N <= 64) { if (spread) KK_LAUNCH(16, 4) else KK_LAUNCH(4, 16) }
+    else { if (spread) KK_LAUNCH(16, 8) else KK_LAUNCH(8, 16) }
+  });
+#undef KK_LAUNCH
+  HIP_CHECK_KERNEL();
+}
+
+}  // namespace kukeon

@@ -268,9 +268,12 @@ def residual_add_rmsnorm(x: torch.Tensor, a, bias, w: torch.Tensor,
 
 
 def clamp_glu(out, gate, up, bg, bu, limit: float, alpha: float,
-              up_shift: float) -> None:
+              up_shift: float, row_scale=None) -> None:
     g = gate.float()
     u = up.float()
+    if row_scale is not None and row_scale.numel():
+        g = g * row_scale[:, None]
+        u = u * row_scale[:, None]
     if bg is not None and bg.numel():
         g = g + bg
         u = u + bu
@@ -404,8 +407,9 @@ def postnorm_residual_rmsnorm(x, y, post_w, w, eps: float, out) -> None:
 
 def conv_act(out, proj, col0: int, cw, bias, state, positions, row_seq,
              cu_rows, state_slots, act: int = 1,
-             shift_state: bool = False) -> None:
-    """out = act(causal_conv(proj[:, col0:col0+C]) + bias) per sequence;
+             shift_state: bool = False, skip: bool = False) -> None:
+    """out = act(causal_conv(proj[:, col0:col0+C]) + bias) per sequence
+    (plus the input itself with `skip`);
     the taps before a portion come from the state slot (zeros before the
     sequence start). cw [taps, C] with the newest tap last. act 1 = silu."""
     taps, C = cw.shape
@@ -429,6 +433,8 @@ def conv_act(out, proj, col0: int, cw, bias, state, positions, row_seq,
         y = y + bias
         if act == 1:
             y = y * torch.sigmoid(y)
+        if skip:
+            y = y + u
         out[r0:r1] = y.to(out.dtype)
         if shift_state and back:
             assert n == 1
@@ -964,3 +970,187 @@ def router_select(idx, wts, logits, top: int, groups: int, keep: int,
     if dense_rows:
         ix = ix * dense_rows + torch.arange(T)[:, None]
     idx[:, :top] = ix.to(idx.dtype)
+
+
+# ---- delta group -----------------------------------------------------------
+def _run_norm(x: torch.Tensor, w: torch.Tensor, groups: int, eps: float):
+    T, W = x.shape
+    return _unit_rms(x.view(T, groups, W // groups), eps).view(T, W) * w
+
+
+def postnorm_residual(x, y, alpha: float, scale, w, groups: int, eps: float,
+                      positions, next: int, h, w2, cw, state,
+                      state_slots) -> None:
+    """x <- norm(alpha x + scale y) * w in runs; next 1: h = x + conv(x) with
+    the state slots shifted (one row per sequence); next 2: h = norm(x) w2.
+    Rows at negative positions become zeros."""
+    live = positions >= 0
+    x.copy_(torch.where(live[:, None], _run_norm(
+        alpha * x + scale * y.float(), w, groups, eps), torch.zeros(())))
+    if next == 1:
+        taps = cw.shape[0]
+        T = x.shape[0]
+        ar = torch.arange(T + 1, dtype=torch.int32)
+        h.zero_()
+        conv_act(h, x, 0, cw, torch.zeros(x.shape[1]), state, positions,
+                 ar[:T], ar, state_slots, 0, taps > 1, True)
+    elif next == 2:
+        h.copy_(torch.where(live[:, None], _run_norm(x, w2, groups, eps),
+                            torch.zeros(())).to(h.dtype))
+
+
+def delta_scan(y, qkv, q_col: int, k_col: int, v_col: int, ba, b_col: int,
+               a_col: int, rate, dt_bias, q_scale: float, state, positions,
+               cu_rows, state_slots, H: int, G: int, d: int, dv: int) -> None:
+    """Gated delta rule, one token after the other; state [slots, H, dv, d]
+    holds S^T."""
+    def unit(t):
+        return t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)
+
+    per = H // G
+    for s in range(cu_rows.numel() - 1):
+        r0, r1 = int(cu_rows[s]), int(cu_rows[s + 1])
+        if r1 <= r0:
+            continue
+        if int(positions[r0]) < 0:
+            y[r0:r1] = 0
+            continue
+        n = r1 - r0
+        slot = int(state_slots[s])
+        S = state[slot].transpose(1, 2).clone()              # [H, d, dv]
+        if int(positions[r0]) == 0:
+            S.zero_()
+        rows = qkv[r0:r1].float()
+        q = unit(rows[:, q_col: q_col + G * d].reshape(n, G, d)) * q_scale
+        k = unit(rows[:, k_col: k_col + G * d].reshape(n, G, d))
+        q = q.repeat_interleave(per, 1)
+        k = k.repeat_interleave(per, 1)
+        v = rows[:, v_col: v_col + H * dv].reshape(n, H, dv)
+        b = torch.sigmoid(ba[r0:r1, b_col: b_col + H].float())
+        g = torch.exp(-rate * torch.nn.functional.softplus(
+            ba[r0:r1, a_col: a_col + H].float() + dt_bias, threshold=30.0))
+        for t in range(n):
+            S = g[t][:, None, None] * S
+            u = b[t][:, None] * (v[t] - (S * k[t][:, :, None]).sum(1))
+            S = S + k[t][:, :, None] * u[:, None, :]
+            y[r0 + t] = (S * q[t][:, :, None]).sum(1).reshape(-1)
+        state[slot] = S.transpose(1, 2)
+
+
+def selective_scan(out, x, z, dt, dt_bias, bc, b_col: int, c_col: int, A2, D,
+                   state, positions, cu_rows, state_slots) -> None:
+    """Selective scan with a decay per (channel, state), one token after the
+    other; state [slots, inner, N]; the result is gated by silu(z)."""
+    N = A2.shape[1]
+    for s in range(cu_rows.numel() - 1):
+        r0, r1 = int(cu_rows[s]), int(cu_rows[s + 1])
+        if r1 <= r0:
+            continue
+        if int(positions[r0]) < 0:
+            out[r0:r1] = 0
+            continue
+        slot = int(state_slots[s])
+        S = state[slot].clone()
+        if int(positions[r0]) == 0:
+            S.zero_()
+        for r in range(r0, r1):
+            xv = x[r].float()
+            step = torch.nn.functional.softplus(dt[r].float() + dt_bias,
+                                                threshold=30.0)
+            B = bc[r, b_col: b_col + N].float()
+            C = bc[r, c_col: c_col + N].float()
+            S = torch.exp2(step[:, None] * A2) * S + \
+                (step * xv)[:, None] * B
+            yv = S @ C + D * xv
+            zf = z[r].float()
+            out[r] = (yv * zf * torch.sigmoid(zf)).to(out.dtype)
+        state[slot] = S
+
+
+def head_norm_append(q_out, k_cache, proj, q_col: int, k_col: int, w,
+                     eps: float, positions, row_seq, block_table) -> None:
+    """q_out = q / rms(q) * w per head; key rows to their page unchanged."""
+    G, BS, d = k_cache.shape[1], k_cache.shape[2], k_cache.shape[3]
+    T, Cq = q_out.shape
+    q = proj[:, q_col: q_col + Cq].float().reshape(T, Cq // d, d)
+    q_out.copy_((_unit_rms(q, eps) * w).reshape(T, Cq).to(q_out.dtype))
+    for r in range(T):
+        p = int(positions[r])
+        if p < 0:
+            continue
+        blk = int(block_table[int(row_seq[r]), p // BS])
+        k_cache[blk, :, p % BS] = proj[r, k_col: k_col + G * d].view(G, d)
+
+
+def masked_attention(out, q, k_cache, v_cache, slopes, r1, r2, positions,
+                     row_seq, block_table, H: int, scale: float,
+                     softcap: float, chunk: int, window: int, sink: bool,
+                     key_eps: float) -> None:
+    G, BS, d = k_cache.shape[1], k_cache.shape[2], k_cache.shape[3]
+    own_v = v_cache is not None and v_cache.numel() > 0
+    dv = v_cache.shape[3] if own_v else d
+    for r in range(q.shape[0]):
+        p = int(positions[r])
+        if p < 0:
+            out[r] = 0
+            continue
+        s = int(row_seq[r])
+        lo = p // chunk * chunk if chunk > 0 else 0
+        if window > 0:
+            lo = max(lo, p - window + 1)
+        js = torch.arange(lo, p + 1)
+        blk = block_table[s, (js // BS).long()].long()
+        k = k_cache[blk, :, (js % BS).long()].float()         # [n, G, d]
+        v = v_cache[blk, :, (js % BS).long()].float() if own_v else k
+        if key_eps >= 0:
+            k = _unit_rms(k, key_eps)
+        qr = q[r].float().view(H, d)
+        dist = (p - js).float()
+        for h in range(H):
+            g = h // (H // G)
+            sc = (k[:, g] @ qr[h]) * scale
+            if softcap > 0:
+                sc = softcap * torch.tanh(sc / softcap)
+            if slopes.numel():
+                sc = sc - slopes[h] * dist
+            if r1.numel():
+                sc = sc - r1[h] * torch.log1p(r2[h] * dist)
+            if sink:
+                sc = torch.cat([sc, torch.zeros(1)])
+                w = torch.softmax(sc, -1)[:-1]
+            else:
+                w = torch.softmax(sc, -1)
+            out[r, h * dv:(h + 1) * dv] = (w @ v[:, g]).to(out.dtype)
+
+
+def router_sigmoid(idx, wts, logits, top: int, scale: float) -> None:
+    """The `top` largest logits (ties: the lower index), weights
+    sigmoid(logit) * scale; further columns of idx and wts are left alone."""
+    ix = torch.sort(logits, dim=-1, descending=True,
+                    stable=True).indices[:, :top]
+    wts[:, :top] = torch.sigmoid(logits.gather(1, ix)) * scale
+    idx[:, :top] = ix.to(idx.dtype)
+
+
+def routed_experts(out, h, idx, wts, top: int, w_gu, w_down, limit: float,
+                   alpha: float, shift: float, weigh_input: bool,
+                   extra) -> None:
+    """out[t] = sum_k w_k expert_k(h_t), or sum_k expert_k(w_k h_t), plus
+    extra[t]."""
+    ff, up = w_down.shape[2], w_gu.shape[1] // 2
+    for t in range(h.shape[0]):
+        acc = torch.zeros(h.shape[1])
+        for k in range(top):
+            e = int(idx[t, k])
+            z = w_gu[e].float() @ h[t].float()
+            g, u = z[:ff], z[up: up + ff]
+            if weigh_input:
+                g, u = g * wts[t, k], u * wts[t, k]
+            g = g.clamp(max=limit)
+            u = u.clamp(-limit, limit)
+            a = (g * torch.sigmoid(alpha * g) * (u + shift)).to(h.dtype)
+            y = w_down[e].float() @ a.float()
+            acc = acc + (y if weigh_input else wts[t, k] * y)
+        if extra.numel():
+            acc = acc + extra[t].float()
+        out[t] = acc.to(out.dtype)
