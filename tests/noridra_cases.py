@@ -1,0 +1,1209 @@
+"""Scenarios for the Noridra family, run by the CPU tests (reference ops,
+fp32) and the GPU tests (HIP kernels, fp32 and bf16). Every scenario builds
+a small configuration with random weights, runs it through the engine and
+compares with the plain model in noridra_oracle.py."""
+import math
+
+import torch
+
+import noridra_oracle as oracle
+from bezizen_cases import (_act, _close, _maps, _poison, check, portions,
+                           row_errors, run_schedule, tokens, tol)
+from kukeon_amd.engine.config import EngineConfig, SamplingParams
+from kukeon_amd.engine.engine import LLMEngine
+from kukeon_amd.engine.kv_cache import SequenceKV
+from kukeon_amd.models.noridra import NoridraConfig, NoridraModel
+
+
+def delta(heads=4, kv_heads=2, dim=5, vdim=7, conv=3):
+    return {"type": "delta", "mixer": {
+        "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+        "conv": conv}}
+
+
+def attn(heads=4, kv_heads=2, dim=6, chunk=9, softcap=5.0, scale=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim,
+         "scale": scale if scale is not None else 2.0 * dim ** -0.5}
+    if softcap:
+        m["softcap"] = softcap
+    if chunk:
+        m["mask"] = {"size": chunk}
+    return {"type": "attention", "mixer": m}
+
+
+def mamba(inner=24, state=5, dt_rank=3, conv=2):
+    return {"type": "mamba1", "mixer": {
+        "inner": inner, "state": state, "dt_rank": dt_rank, "conv": conv}}
+
+
+def moe(experts, top, ff):
+    return {"kind": "moe", "expert": {"ff": ff},
+            "router": {"experts": experts, "top": top}}
+
+
+def layer(mix, mlp):
+    return dict(mix, mlp=mlp)
+
+
+def config(layers, width=40, vocab=45, eps=1e-5, groups=5, alpha=1.7, taps=3,
+           positions=400):
+    return {"architecture": "Noridra", "width": width, "vocab": vocab,
+            "norm": {"eps": eps, "groups": groups}, "postln_alpha": alpha,
+            "canon": {"taps": taps}, "max_positions": positions,
+            "layers": layers}
+
+
+CONFIGS = {
+    # all mixers, shared and own key heads, a layer without a feed-forward,
+    # sizes off every vector path
+    "hybrid": lambda: config([
+        layer(delta(), moe(5, 2, 9)),
+        layer(attn(), moe(4, 1, 12)),
+        layer(mamba(), None),
+        layer(delta(heads=3, kv_heads=3, dim=8, vdim=12, conv=2),
+              moe(3, 3, 10)),
+        layer(mamba(inner=17, state=3, dt_rank=20, conv=4), moe(6, 2, 7)),
+    ]),
+    # rows of whole 16-byte pieces everywhere (the vector forms), four query
+    # heads on one kv head, state rows over several lanes
+    "aligned": lambda: config([
+        layer(delta(heads=4, kv_heads=2, dim=64, vdim=40, conv=4),
+              moe(4, 1, 64)),
+        layer(attn(heads=4, kv_heads=1, dim=16, chunk=20, softcap=30.0),
+              moe(8, 2, 64)),
+        layer(mamba(inner=192, state=16, dt_rank=16, conv=4), moe(4, 3, 32)),
+        layer(delta(heads=2, kv_heads=2, dim=128, vdim=64, conv=2), None),
+    ], width=128, vocab=50, eps=1e-3, groups=4, taps=4),
+    # everything at its simplest: one run in the norm, unit factor, one tap
+    # everywhere, no chunk, no cap, one head, a width off multiples of 8, one
+    # expert, no position table
+    "plain": lambda: config([
+        layer(attn(heads=1, kv_heads=1, dim=7, chunk=0, softcap=0),
+              moe(1, 1, 5)),
+        layer(mamba(inner=9, state=1, dt_rank=1, conv=1), None),
+        layer(delta(heads=1, kv_heads=1, dim=3, vdim=1, conv=1),
+              moe(2, 2, 11)),
+    ], width=26, vocab=31, groups=1, alpha=1.0, taps=1, positions=0),
+    # runs of one entry, chunks of one token
+    "extreme": lambda: config([
+        layer(attn(heads=2, kv_heads=1, dim=8, chunk=1), moe(3, 2, 8)),
+        layer(delta(heads=6, kv_heads=2, dim=4, vdim=9, conv=5), None),
+    ], width=16, vocab=21, groups=16, alpha=0.5, taps=6),
+    "only_delta": lambda: config([
+        layer(delta(heads=2, kv_heads=1, dim=4, vdim=8), moe(3, 2, 8)),
+        layer(delta(heads=1, kv_heads=1, dim=40, vdim=3), None),
+    ], width=16, vocab=21, groups=2),
+    "only_mamba": lambda: config([
+        layer(mamba(inner=32, state=8, dt_rank=4, conv=3), None),
+    ], width=16, vocab=21, groups=2, taps=2),
+    "only_attention": lambda: config([
+        layer(attn(heads=2, kv_heads=2, dim=8, chunk=300), None),
+        layer(attn(heads=3, kv_heads=1, dim=8, chunk=4), moe(3, 2, 8)),
+    ], width=16, vocab=21, groups=8, taps=5),
+    # long key rows and wide state rows
+    "wide": lambda: config([
+        layer(delta(heads=2, kv_heads=1, dim=160, vdim=20, conv=2), None),
+        layer(mamba(inner=40, state=40, dt_rank=5, conv=3), None),
+        layer(delta(heads=1, kv_heads=1, dim=260, vdim=18, conv=4),
+              moe(2, 1, 16)),
+        layer(mamba(inner=24, state=70, dt_rank=8, conv=2), None),
+    ], width=32, vocab=40, groups=4),
+    # heads of 128 on pages of 16: the sizes of the matrix-core attention
+    # kernel that long portions take; a chunk that ends inside a key tile,
+    # three query heads per kv head
+    "tiles": lambda: config([
+        layer(attn(heads=6, kv_heads=2, dim=128, chunk=40, softcap=8.0,
+                   scale=0.12), moe(4, 2, 16)),
+        layer(mamba(inner=64, state=16, dt_rank=8, conv=4), None),
+        layer(attn(heads=3, kv_heads=1, dim=128, chunk=0, softcap=0,
+                   scale=0.1), None),
+    ], width=48, vocab=40, groups=3),
+    # a chunk longer than one pass of the attention kernel over the keys
+    "long_chunk": lambda: config([
+        layer(attn(heads=2, kv_heads=1, dim=8, chunk=150, softcap=20.0,
+                   scale=0.9), None),
+        layer(delta(heads=2, kv_heads=2, dim=8, vdim=8), moe(4, 2, 8)),
+    ], width=16, vocab=19, groups=2),
+}
+
+
+def weights(cfg, seed=0):
+    """Random checkpoint for a config dictionary, bf16 like a stored one."""
+    g = torch.Generator().manual_seed(seed)
+    W, V = cfg["width"], cfg["vocab"]
+
+    def r(*shape, std=1.0, mean=0.0):
+        return (torch.randn(*shape, generator=g) * std + mean).to(
+            torch.bfloat16)
+
+    t = {"embed": r(V, W), "final.norm": r(W, std=0.2, mean=1.0),
+         "head": r(V, W, std=W ** -0.5)}
+    if cfg.get("max_positions"):
+        t["pos"] = r(cfg["max_positions"], W, std=0.5)
+    for i, L in enumerate(cfg["layers"]):
+        p = "l%d." % i
+        m = L["mixer"]
+        for q in ("1", "2") if L["mlp"] else ("1",):
+            t[p + "norm" + q] = r(W, std=0.2, mean=1.0)
+            t[p + "ls" + q] = r(W, std=0.2, mean=0.7)
+            t[p + "canon" + q] = r(W, cfg["canon"]["taps"], std=0.4)
+        q = p + "mix."
+        if L["type"] == "delta":
+            H, G, D, U = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            for n, c in (("q", G * D), ("k", G * D), ("v", H * U)):
+                t[q + n] = r(c, W, std=1.5 * W ** -0.5)
+                t[q + n + ".conv"] = r(c, m["conv"], std=0.5, mean=0.4)
+            t[q + "b"] = r(H, W, std=W ** -0.5)
+            t[q + "a"] = r(H, W, std=W ** -0.5)
+            t[q + "A_log"] = r(H, std=0.7, mean=-1.0)
+            t[q + "dt_bias"] = r(H, std=0.7, mean=-1.0)
+            t[q + "norm"] = r(U, std=0.2, mean=1.0)
+            t[q + "g"] = r(H * U, W, std=2.0 * W ** -0.5)
+            t[q + "o"] = r(W, H * U, std=(H * U) ** -0.5)
+        elif L["type"] == "attention":
+            Cq, Ck = m["heads"] * m["dim"], m["kv_heads"] * m["dim"]
+            t[q + "q"] = r(Cq, W, std=W ** -0.5)
+            t[q + "k"] = r(Ck, W, std=1.5 * W ** -0.5)
+            t[q + "q.norm"] = r(m["dim"], std=0.3, mean=1.2)
+            t[q + "k.norm"] = r(m["dim"], std=0.3, mean=0.8)
+            t[q + "r1"] = r(m["heads"], std=0.1, mean=0.5)
+            t[q + "r2"] = (torch.rand(m["heads"], generator=g) + 0.2).to(
+                torch.bfloat16)
+            t[q + "g"] = r(Cq, W, std=2.0 * W ** -0.5)
+            t[q + "o"] = r(W, Cq, std=Cq ** -0.5)
+        else:
+            I, N, R = m["inner"], m["state"], m["dt_rank"]
+            t[q + "in"] = r(2 * I, W, std=W ** -0.5)
+            t[q + "conv"] = r(I, m["conv"], std=0.4, mean=0.4)
+            t[q + "conv.b"] = r(I, std=0.3)
+            t[q + "x"] = r(R + 2 * N, I, std=I ** -0.5)
+            t[q + "dt"] = r(I, R, std=R ** -0.5)
+            t[q + "dt.b"] = r(I, std=0.7, mean=-1.5)
+            t[q + "A_log"] = r(I, N, std=0.7)
+            t[q + "D"] = r(I, std=0.3, mean=0.5)
+            t[q + "o"] = r(W, I, std=I ** -0.5)
+        f = L["mlp"]
+        if not f:
+            continue
+        q = p + "mlp."
+        E, ff = f["router"]["experts"], f["expert"]["ff"]
+        t[q + "router"] = r(E, W, std=2.0 * W ** -0.5)
+        for e in range(E):
+            t[q + f"e{e}.gate"] = r(ff, W, std=2.0 * W ** -0.5)
+            t[q + f"e{e}.up"] = r(ff, W, std=2.0 * W ** -0.5)
+            t[q + f"e{e}.down"] = r(W, ff, std=ff ** -0.5)
+    return t
+
+
+def make_engine(cfg, tensors, device, dtype, blocks=96, slots=4,
+                block_size=4, max_len=384, poison=True, **ekw):
+    mcfg = NoridraConfig.from_json(cfg)
+    model = NoridraModel(mcfg, device=device, dtype=dtype, tensors=tensors,
+                         max_position=max_len)
+    kw = dict(block_size=block_size, max_model_len=max_len,
+              max_sessions=slots, state_slots=slots, num_kv_blocks=blocks,
+              use_graphs=False)
+    kw.update(ekw)
+    eng = LLMEngine(model, mcfg, EngineConfig(**kw), device=device)
+    if poison:
+        _poison(eng)
+    return eng
+
+
+def logits_of(cfg, W, toks):
+    return oracle.forward(toks, W, cfg)
+
+
+# ---------------------------------------------------------------- scenarios
+def case_whole(name, device, dtype, n=27):
+    cfg = CONFIGS[name]()
+    W = weights(cfg, 1)
+    toks = tokens(cfg, n, 1)
+    eng = make_engine(cfg, W, device, dtype,
+                      block_size=16 if name == "tiles" else 4)
+    got = run_schedule(eng, [toks], [[(0, len(toks))]])[0]
+    check(got, logits_of(cfg, W, toks), dtype, name)
+
+
+def case_layers(device, dtype):
+    """The residual stream after every layer."""
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 2)
+    toks = tokens(cfg, 11, 2)
+    eng = make_engine(cfg, W, device, dtype)
+    want = []
+    oracle.forward(toks, W, cfg, want)
+    kv = SequenceKV(eng.ecfg.block_size)
+    got = []
+    fwd = eng.model.forward
+    eng.model.forward = lambda *a, **k: fwd(*a, taps=got, **k)
+    eng.forward_tokens([(kv, toks)])
+    eng.model.forward = fwd
+    assert len(got) == len(want) == len(cfg["layers"])
+    for i, (g, w) in enumerate(zip(got, want)):
+        e = row_errors(g, w)
+        over = int((e > tol(dtype)).sum())
+        assert over <= (0 if dtype == "fp32" else 1), \
+            f"layer {i}: {float(e.max()):.3g}"
+
+
+def case_prefill_vs_decode(name, device, dtype):
+    cfg = CONFIGS[name]()
+    W = weights(cfg, 3)
+    toks = tokens(cfg, 25, 3)
+    want = logits_of(cfg, W, toks)
+    whole = run_schedule(make_engine(cfg, W, device, dtype), [toks],
+                         [[(0, len(toks))]])[0]
+    one = run_schedule(make_engine(cfg, W, device, dtype), [toks],
+                       [[(0, 1)] for _ in toks])[0]
+    check(whole, want, dtype, "whole")
+    check(one, want, dtype, "token by token")
+    check(one, whole, dtype, "token by token against whole")
+
+
+def case_portions(name, device, dtype, sizes, n=41):
+    cfg = CONFIGS[name]()
+    W = weights(cfg, 4)
+    toks = tokens(cfg, n, 4)
+    sched = [[(0, k)] for k in portions(len(toks), sizes)]
+    got = run_schedule(make_engine(cfg, W, device, dtype), [toks], sched)[0]
+    check(got, logits_of(cfg, W, toks), dtype, f"portions {sizes}")
+
+
+def case_batch(name, device, dtype):
+    """Unequal requests in one batch, portions beside single tokens."""
+    cfg = CONFIGS[name]()
+    W = weights(cfg, 5)
+    prompts = [tokens(cfg, n, 10 + n) for n in (19, 1, 7, 30)]
+    sched = [
+        [(0, 5), (1, 1), (3, 2)],
+        [(0, 1), (2, 7), (3, 9)],
+        [(3, 1), (0, 1)],
+        [(0, 12), (3, 1)],
+        [(3, 17)],
+    ]
+    got = run_schedule(make_engine(cfg, W, device, dtype), prompts, sched)
+    for i, p in enumerate(prompts):
+        alone = run_schedule(make_engine(cfg, W, device, dtype), [p],
+                             [[(0, len(p))]])[0]
+        check(got[i], logits_of(cfg, W, p), dtype, f"request {i}")
+        check(got[i], alone, dtype, f"request {i} against itself alone")
+
+
+def case_reuse(device, dtype):
+    """A pool too small for all requests at once: pages and state slots of
+    finished requests are handed to the next ones."""
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 6)
+    prompts = [tokens(cfg, n, 20 + n) for n in (14, 11, 16, 3, 13)]
+    eng = make_engine(cfg, W, device, dtype, blocks=8, slots=2, block_size=4)
+    sched = [
+        [(0, 6), (1, 4)],
+        [(0, 8), (1, 1)],          # 0 ends: 4 pages and a slot come back
+        [(1, 6), (2, 9)],          # 1 ends
+        [(2, 7), (3, 2)],          # 2 ends
+        [(3, 1), (4, 12)],         # 3 ends
+        [(4, 1)],
+    ]
+    got = run_schedule(eng, prompts, sched)
+    for i, p in enumerate(prompts):
+        check(got[i], logits_of(cfg, W, p), dtype, f"request {i}")
+    assert eng.kv.allocator.num_free == 8 and eng.states.num_free == 2
+
+
+def case_first_tokens(device, dtype):
+    """Short sequences started in used pages and slots, and a start cut
+    into single tokens."""
+    for name in ("hybrid", "extreme"):
+        cfg = CONFIGS[name]()
+        W = weights(cfg, 7)
+        eng = make_engine(cfg, W, device, dtype, slots=1)
+        for n, sched in ((1, [1]), (2, [2]), (3, [1, 2]),
+                         (9, [1, 1, 1, 2, 4]), (6, [2, 1, 3])):
+            toks = tokens(cfg, n, 30 + n)
+            got = run_schedule(eng, [toks], [[(0, k)] for k in sched])[0]
+            check(got, logits_of(cfg, W, toks), dtype, f"{name} {n}")
+
+
+def case_long_decode(device, dtype):
+    """Decoding past the chunks and through many pages."""
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 8)
+    toks = tokens(cfg, 75, 8)
+    sched = [[(0, 3)]] + [[(0, 1)] for _ in range(72)]
+    got = run_schedule(make_engine(cfg, W, device, dtype, block_size=4),
+                       [toks], sched)[0]
+    check(got, logits_of(cfg, W, toks), dtype, "long decode")
+
+
+def case_long_chunk(device, dtype):
+    """A chunk longer than one pass of the attention kernel over the keys,
+    a prompt of several chunks, portions that end inside one."""
+    cfg = CONFIGS["long_chunk"]()
+    W = weights(cfg, 9)
+    toks = tokens(cfg, 330, 9)
+    want = logits_of(cfg, W, toks)
+    eng = make_engine(cfg, W, device, dtype, blocks=200, max_len=400)
+    got = run_schedule(eng, [toks], [[(0, 330)]])[0]
+    check(got, want, dtype, "whole")
+    sched = [[(0, 149)], [(0, 2)], [(0, 146)]] + [[(0, 1)]] * 33
+    got = run_schedule(eng, [toks], sched)[0]
+    check(got, want, dtype, "portions and decoding")
+
+
+def case_long_portions(device, dtype):
+    """Portions long enough for the matrix-core attention kernel beside
+    single tokens, cut inside a chunk and inside a key tile."""
+    cfg = CONFIGS["tiles"]()
+    W = weights(cfg, 13)
+    prompts = [tokens(cfg, n, 80 + n) for n in (150, 61, 40)]
+    want = [logits_of(cfg, W, p) for p in prompts]
+    eng = make_engine(cfg, W, device, dtype, blocks=40, block_size=16,
+                      max_len=256)
+    sched = [
+        [(0, 70), (1, 20)],
+        [(0, 1), (1, 41), (2, 39)],
+        [(0, 45), (2, 1)],
+        [(0, 34)],
+    ]
+    got = run_schedule(eng, prompts, sched)
+    for i in range(3):
+        check(got[i], want[i], dtype, f"request {i}")
+
+
+def case_sorted_experts(device, dtype):
+    """Long portions sort their rows by expert and run each expert over its
+    rows at once; short steps take the pair kernels. Both against the plain
+    model, two requests in the long step."""
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 12)
+    prompts = [tokens(cfg, n, 70 + n) for n in (90, 71)]
+    want = [logits_of(cfg, W, p) for p in prompts]
+    eng = make_engine(cfg, W, device, dtype, blocks=64, max_len=128)
+    got = run_schedule(eng, prompts, [[(0, 90), (1, 70)], [(1, 1)]])
+    for i in range(2):
+        check(got[i], want[i], dtype, f"sorted rows, request {i}")
+
+
+def case_generate(device, dtype, use_graphs=False):
+    """Greedy generation through add_request / step against greedy decoding
+    with the plain model (a token whose two best logits nearly tie in the
+    plain model may differ: generation is compared up to the first such
+    place)."""
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 10)
+    prompts = [tokens(cfg, n, 50 + n) for n in (9, 4, 13)]
+    new = 12
+    eng = make_engine(cfg, W, device, dtype, use_graphs=use_graphs,
+                      graph_buckets=(4,), decode_microbatch=4)
+    sp = SamplingParams(temperature=0.0, top_k=1, top_p=1.0,
+                        max_new_tokens=new)
+    kvs = [SequenceKV(eng.ecfg.block_size) for _ in prompts]
+    rids = [eng.add_request(kv, p, sp) for kv, p in zip(kvs, prompts)]
+    outs = {r: [] for r in rids}
+    for _ in range(200):
+        if not eng.has_work():
+            break
+        for o in eng.step():
+            outs[o.req_id].extend(o.new_tokens)
+    assert not eng.has_work()
+    margin = 0.02 if dtype == "fp32" else 0.6
+    for rid, p in zip(rids, prompts):
+        got = outs[rid]
+        assert len(got) == new
+        seq = list(p)
+        for k in range(new):
+            lg = logits_of(cfg, W, seq)[-1]
+            top2 = lg.topk(2).values
+            if float(top2[0] - top2[1]) < margin:
+                break
+            assert got[k] == int(lg.argmax()), f"request {rid}, token {k}"
+            seq.append(got[k])
+    for kv in kvs:
+        eng.free_sequence(kv)
+    assert eng.kv.allocator.num_free == eng.kv.num_blocks
+
+
+def case_graph_replays(device, dtype):
+    """Steps under captured graphs against the same steps run eagerly: the
+    logits path is the same, so with equal seeds the sampled tokens are."""
+    cfg = CONFIGS["aligned"]()
+    W = weights(cfg, 17)
+    prompts = [tokens(cfg, n, 90 + n) for n in (21, 5)]
+    outs = []
+    for graphs in (False, True):
+        eng = make_engine(cfg, W, device, dtype, use_graphs=graphs,
+                          graph_buckets=(4,), decode_microbatch=3)
+        got = []
+        for turn in range(3):            # eager work between the replays
+            kvs = [SequenceKV(eng.ecfg.block_size) for _ in prompts]
+            sp = SamplingParams(temperature=0.0, top_k=1, top_p=1.0,
+                                max_new_tokens=10)
+            rids = [eng.add_request(kv, p[turn:], sp)
+                    for kv, p in zip(kvs, prompts)]
+            res = {r: [] for r in rids}
+            while eng.has_work():
+                for o in eng.step():
+                    res[o.req_id].extend(o.new_tokens)
+            got += [res[r] for r in rids]
+            for kv in kvs:
+                eng.free_sequence(kv)
+        outs.append(got)
+    # graphs pad the batch to a bucket, which may reorder a few sums of the
+    # library's products, so late tokens may part after a close call
+    same = sum(a[k] == b[k] for a, b in zip(*outs) for k in range(10))
+    assert same >= 0.8 * 10 * len(outs[0]), f"{same} of {10 * len(outs[0])}"
+    assert all(a[0] == b[0] for a, b in zip(*outs))
+
+
+def assert_greedy(cfg, W, prompt, got, what=""):
+    """Every generated token is the plain model's best one, up to the
+    rounding of the logits to bfloat16 that the sampler works on."""
+    toks = list(prompt)
+    for i, t in enumerate(got):
+        lg = logits_of(cfg, W, toks)[-1]
+        best = float(lg.max())
+        slack = abs(best) * 2.0 ** -7
+        assert float(lg[t]) >= best - slack, \
+            f"{what}: token {i} is {t}, the plain model says " \
+            f"{int(lg.argmax())}"
+        toks.append(t)
+
+
+def _generate(eng, kv, prompt, n):
+    sp = SamplingParams(temperature=0.0, max_new_tokens=n)
+    eng.add_request(kv, prompt, sp)
+    out = []
+    while eng.has_work():
+        for o in eng.step():
+            out.extend(o.new_tokens)
+    return out
+
+
+def case_multi_turn(device):
+    """A session's second turn continues from its pages and state slot; an
+    idle session whose pages and slot were taken away is rebuilt from its
+    history."""
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 15)
+    eng = make_engine(cfg, W, device, "fp32", blocks=12, slots=2, max_len=64,
+                      poison=False, decode_microbatch=2)
+    a, b = SequenceKV(4), SequenceKV(4)
+    p1, p2, p3 = tokens(cfg, 9, 60), tokens(cfg, 5, 61), tokens(cfg, 30, 62)
+    t1 = _generate(eng, a, p1, 4)
+    assert_greedy(cfg, W, p1, t1, "first turn")
+    t2 = _generate(eng, a, p2, 3)
+    assert_greedy(cfg, W, p1 + t1 + p2, t2, "second turn")
+    assert a.num_tokens > 0 and a.state_slot >= 0
+    tb = _generate(eng, b, p3, 4)       # needs a's pages
+    assert_greedy(cfg, W, p3, tb, "other session")
+    assert a.num_tokens == 0 and a.state_slot < 0 and a.history
+    eng.free_sequence(b)
+    t3 = _generate(eng, a, [7, 3], 3)
+    assert_greedy(cfg, W, p1 + t1 + p2 + t2 + [7, 3], t3, "rebuilt session")
+
+
+# ----------------------------------------------------- mechanisms, one by one
+def _pointing(chunk, dim, scale, taps=2, softcap=0.0):
+    """A one-layer stack whose token 8 a + b asks for keys of kind a and is
+    itself a key of kind b; the norms and the input convolution are made
+    neutral, so that a score stands out by `scale` alone."""
+    cfg = config([layer(attn(heads=2, kv_heads=1, dim=dim, chunk=chunk,
+                             scale=scale, softcap=softcap), None)],
+                 width=16, vocab=64, groups=1, alpha=1.0, taps=taps,
+                 positions=0)
+    W = weights(cfg, 20)
+    V, Wd = 64, 16
+    emb = torch.zeros(V, Wd)
+    for v in range(V):
+        emb[v, v % 8] = 1.0
+        emb[v, 8 + v // 8] = 1.0
+    b = lambda t: t.to(torch.bfloat16)
+    W["embed"] = b(emb)
+    W["l0.canon1"] = b(torch.zeros(Wd, taps))
+    W["l0.norm1"] = b(torch.ones(Wd))
+    W["l0.ls1"] = b(torch.ones(Wd))
+    wq, wk = torch.zeros(2 * dim, Wd), torch.zeros(dim, Wd)
+    for a in range(8):
+        wq[a, 8 + a] = 1.0
+        wq[dim + a, 8 + a] = 1.0
+        wk[a, a] = 1.0
+    W["l0.mix.q"], W["l0.mix.k"] = b(wq), b(wk)
+    W["l0.mix.q.norm"] = b(torch.ones(dim))
+    W["l0.mix.k.norm"] = b(torch.ones(dim))
+    return cfg, W
+
+
+def case_chunk_edges(device, dtype, decode, dim=8, bs=4):
+    """One key that the queries point at: the first and the last of a chunk,
+    at a page border, position 0, the query's own. Values are the keys, so
+    with the key visible the output is (close to) that key's row; from the
+    next chunk on it is hidden."""
+    chunk = 10
+    cfg, W = _pointing(chunk, dim, 12.0 / dim)
+    W["l0.mix.r1"] = torch.zeros(2).to(torch.bfloat16)
+    n = 3 * chunk + 5
+    for target in (0, 3, bs * 2 - 1, bs * 2, chunk - 1, chunk, 2 * chunk,
+                   n - 1):
+        toks = [8 * 1 + 0] * n
+        toks[target] = 8 * 1 + 1
+        want = logits_of(cfg, W, toks)
+        eng = make_engine(cfg, W, device, dtype, block_size=bs)
+        if decode:
+            sched = [[(0, 2)]] + [[(0, 1)]] * (n - 2)
+        else:
+            sched = [[(0, n - 17)], [(0, 17)]]
+        got = run_schedule(eng, [toks], sched)[0]
+        check(got, want, dtype, f"key {target}")
+        last_seen = target // chunk * chunk + chunk - 1
+        if target < last_seen and last_seen + 1 < n:
+            a, b = want[last_seen], want[last_seen + 1]
+            assert float((a - b).abs().max()) > 0.05
+
+
+def case_far_key(device, dtype, decode):
+    """One key hundreds of positions back that the queries point at, under a
+    distance bias that matters but does not hide it; the first key of all,
+    and one at a page border."""
+    cfg, W = _pointing(0, 8, 0.8)
+    W["l0.mix.r1"] = torch.tensor([0.4, 1.0]).to(torch.bfloat16)
+    W["l0.mix.r2"] = torch.tensor([0.5, 2.0]).to(torch.bfloat16)
+    n = 300
+    for target in (0, 63, 64):
+        toks = [8 + 0] * n
+        toks[target] = 8 + 1
+        want = logits_of(cfg, W, toks)
+        eng = make_engine(cfg, W, device, dtype, block_size=16, max_len=320)
+        sched = ([[(0, n - 12)]] + [[(0, 1)]] * 12 if decode
+                 else [[(0, 130)], [(0, 170)]])
+        got = run_schedule(eng, [toks], sched)[0]
+        check(got, want, dtype, f"key {target}")
+        # the key is seen, and the bias counts
+        hidden = logits_of(cfg, W, [8 + 0] * n)
+        assert float((want[-1] - hidden[-1]).abs().max()) > 0.02
+        flat = dict(W)
+        flat["l0.mix.r1"] = torch.zeros(2)
+        assert float((want[-1] - logits_of(cfg, flat, toks)[-1]).abs()
+                     .max()) > 0.02
+
+
+def case_sink(device, dtype):
+    """Scores far below zero: nearly all weight sits on the sink and the
+    attention's output nearly vanishes; and scores far above, where the sink
+    must not matter. Without the sink the first would be a plain average."""
+    for scale, small in ((-30.0, True), (-2.0, True), (30.0, False)):
+        cfg, W = _pointing(0, 8, scale / 8.0)
+        toks = [8 + 1] * 20
+        want = logits_of(cfg, W, toks)
+        t64 = {k: v.double() for k, v in W.items()}
+        h = oracle.embed(toks, t64)
+        m = dict(cfg["layers"][0]["mixer"])
+        out = oracle.attention_mixer(h, t64, "l0.mix.", m, 1e-5)
+        ref = oracle.attention_mixer(h, t64, "l0.mix.", dict(m, scale=4.0),
+                                     1e-5)
+        assert (float(out.abs().max()) < 0.9 * float(ref.abs().max())) == small
+        eng = make_engine(cfg, W, device, dtype)
+        got = run_schedule(eng, [toks], [[(0, 17)], [(0, 1)], [(0, 1)],
+                                         [(0, 1)]])[0]
+        check(got, want, dtype, f"scale {scale}")
+
+
+def case_state_carry(device, dtype):
+    """Both recurrences with decays pushed to (nearly) one: what the first
+    tokens wrote must survive every cut and reach the last position."""
+    for kind in ("delta", "mamba1"):
+        mix = delta(heads=2, kv_heads=1, dim=64, vdim=8, conv=3) \
+            if kind == "delta" else mamba(inner=32, state=8, dt_rank=4, conv=3)
+        cfg = config([layer(mix, None)], width=16, vocab=32, groups=2,
+                     alpha=0.5, positions=0)
+        W = weights(cfg, 22)
+        W["l0.mix.A_log"] = torch.full_like(W["l0.mix.A_log"], -9.0)
+        n = 100
+        toks = tokens(cfg, n, 22)
+        if kind == "delta":
+            # later keys must not erase what the first one wrote
+            W["l0.mix.b"] = torch.zeros_like(W["l0.mix.b"])
+        want = logits_of(cfg, W, toks)
+        other = [(toks[0] + 1) % cfg["vocab"]] + toks[1:]
+        far = logits_of(cfg, W, other)
+        assert float((far[-1] - want[-1]).abs().max()) > 0.01
+        eng = make_engine(cfg, W, device, dtype, blocks=64, max_len=128)
+        for sched in ([n], [1, 2, 50] + [1] * 47, [30, 33, 2, 35]):
+            got = run_schedule(eng, [toks], [[(0, k)] for k in sched])[0]
+            check(got, want, dtype, f"{kind}, cuts {sched[:4]}")
+
+
+def case_input_conv(device, dtype):
+    """The sublayers' input convolution: a token just inside its reach moves
+    the logits through it, one just outside does not (single mixer without
+    any other memory: chunks of one token)."""
+    cfg = config([layer(attn(heads=1, kv_heads=1, dim=8, chunk=1), None)],
+                 width=16, vocab=24, groups=2, taps=4, positions=0)
+    W = weights(cfg, 24)
+    W["l0.canon1"] = (W["l0.canon1"].float() * 3).to(torch.bfloat16)
+    toks = tokens(cfg, 12, 24)
+    want = logits_of(cfg, W, toks)
+    for back, seen in ((3, True), (4, False)):
+        other = list(toks)
+        other[11 - back] = (other[11 - back] + 1) % 24
+        d = float((logits_of(cfg, W, other)[-1] - want[-1]).abs().max())
+        assert (d > 1e-3) == seen
+    eng = make_engine(cfg, W, device, dtype)
+    for sched in ([12], [1] * 12, [2, 1, 2, 3, 1, 3], [4, 8], [11, 1]):
+        got = run_schedule(eng, [toks], [[(0, k)] for k in sched])[0]
+        check(got, want, dtype, f"cuts {sched}")
+
+
+def case_router(device, dtype):
+    """Routed experts alone against the plain model: every `top`, rows in
+    both forms of the expert pass, on and off the matrix-core sizes."""
+    from kukeon_amd.models.feedforward import RoutedMoE
+    for E, top, ff, Wd, T in ((6, 2, 10, 24, 5), (8, 3, 24, 40, 70),
+                              (4, 4, 8, 24, 66), (5, 1, 9, 22, 3),
+                              (3, 2, 72, 136, 40), (2, 2, 64, 256, 63)):
+        f = moe(E, top, ff)
+        cfg = config([layer(mamba(), f)], width=Wd, groups=1)
+        W = weights(cfg, 30 + E)
+        t64 = {k: v.double() for k, v in W.items()}
+        g = torch.Generator().manual_seed(E)
+        h = torch.randn(T, Wd, generator=g).to(torch.bfloat16)
+        want = oracle.moe(h.double(), t64, "l0.mlp.", f)
+        fc = NoridraConfig.from_json(cfg).layers[0].mlp
+        mod = RoutedMoE(fc, Wd, W, "l0.mlp.", device, _act(dtype))
+
+        class Meta:
+            host_ids = list(range(T))
+        for meta in (Meta(), None):
+            got = mod(h.to(device=device, dtype=_act(dtype)), None, meta)
+            check(got, want, dtype, f"experts {E} top {top}")
+
+
+# ------------------------------------------------------- single operations
+def case_op_postnorm(device, dtype):
+    """The norm after the sum, alone, with the next input's convolution and
+    with a second norm; an inactive row among live ones."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(5)
+    for Wd, groups, taps in ((16, 1, 1), (40, 5, 3), (128, 4, 4), (26, 2, 2),
+                             (26, 26, 6), (4096, 4, 4), (2048, 64, 3)):
+        T, eps, alpha = 5, 1e-4, 1.3
+        x = torch.randn(T, Wd, generator=g)
+        y = torch.randn(T, Wd, generator=g).to(_act(dtype))
+        ls, w, w2 = (torch.randn(Wd, generator=g) for _ in range(3))
+        cw = torch.randn(taps, Wd, generator=g)
+        st0 = torch.randn(6, taps - 1, Wd, generator=g)
+        pos = [7, 0, -1, 1, 30]
+        slots = [4, 0, 1, 2, 5]
+        cfg = {"norm": {"groups": groups, "eps": eps}}
+        want = oracle.group_norm(alpha * x.double() + ls.double() *
+                                 y.double(), w.double(), cfg)
+        want[2] = 0
+        conv = want.clone()
+        for r in range(T):
+            if pos[r] < 0:
+                continue
+            for j in range(taps):
+                if pos[r] - (taps - 1) + j < 0:
+                    continue
+                u = want[r] if j == taps - 1 else st0[slots[r], j].double()
+                conv[r] += cw[j].double() * u
+        second = oracle.group_norm(want, w2.double(), cfg)
+        second[2] = 0
+        d = lambda t: t.to(device)
+        i32 = lambda t: torch.tensor(t, dtype=torch.int32, device=device)
+        args = (d(y), alpha, d(ls), d(w), groups, eps, i32(pos))
+        xd = d(x.clone())
+        ops.postnorm_residual(xd, *args)
+        _close(xd, want, "fp32", f"{Wd}: norm")
+        xd, st = d(x.clone()), d(st0.clone())
+        h = torch.full((T, Wd), 9.0, dtype=_act(dtype), device=device)
+        ops.postnorm_residual_conv(xd, *args, h, d(cw), st, i32(slots))
+        _close(xd, want, "fp32", f"{Wd}: norm before the convolution")
+        _close(h, conv, dtype, f"{Wd}: convolution")
+        moved = st0.double().clone()
+        for r in range(T):
+            if pos[r] >= 0 and taps > 1:
+                moved[slots[r]] = torch.cat([st0[slots[r]].double(),
+                                             want[r][None]])[1:]
+        if taps > 1:
+            _close(st, moved, "fp32", f"{Wd}: tails")
+        xd = d(x.clone())
+        h = torch.full((T, Wd), 9.0, dtype=_act(dtype), device=device)
+        ops.postnorm_residual_norm(xd, *args, h, d(w2))
+        _close(h, second, dtype, f"{Wd}: second norm")
+
+
+def case_op_conv(device, dtype):
+    """The convolution with the input added, fp32 rows in and activations
+    out, over portions long enough for the run form: sequences that begin
+    inside a run, a dirty slot, an inactive neighbour."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(6)
+    for Wd, taps, cuts in ((24, 4, (45, 1, 30)), (64, 3, (70, 9, 2)),
+                           (40, 2, (64, 64)), (16, 5, (3, 80)),
+                           (22, 3, (40, 40)), (1024, 4, (33, 50))):
+        total = sum(cuts)
+        cw = torch.randn(taps, Wd, generator=g)
+        bias = torch.randn(Wd, generator=g)
+        seqs = [torch.randn(total, Wd, generator=g) for _ in range(2)]
+        for act, skip in ((0, True), (1, False)):
+            state = torch.full((4, taps - 1, Wd), -700.0, device=device)
+            zero = torch.zeros(Wd, device=device)
+            got, at = [[], []], 0
+            for n in cuts:
+                u = torch.cat([seqs[0][at: at + n], torch.ones(3, Wd),
+                               seqs[1][at: at + n]]).to(device)
+                pos, row_seq, cu, slots = _maps([n, 3, n], [at, -1, at],
+                                                device, [2, 1, 0])
+                out = torch.full(u.shape, 9.0, dtype=_act(dtype),
+                                 device=device)
+                ops.conv_act(out, u, 0, cw.to(device), bias.to(device), state,
+                             pos, row_seq, cu, slots, act, False, skip)
+                ops.conv_tail_update(state, u, 0, zero, pos, cu, slots)
+                got[0].append(out[:n])
+                got[1].append(out[n + 3:])
+                at += n
+            for k in range(2):
+                want = oracle.short_conv(seqs[k].double(), cw.double().T) + \
+                    bias.double()
+                if act:
+                    want = oracle.silu(want)
+                if skip:
+                    want = want + seqs[k].double()
+                _close(torch.cat(got[k]), want, dtype, f"{Wd} {act} {k}")
+
+
+def case_op_delta(device, dtype, H=4, G=2, d=5, dv=7, cuts=(4, 1, 9, 1, 1)):
+    """The delta rule over portions with a dirty slot and an inactive
+    neighbour."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(7 + d)
+    n = sum(cuts)
+    act = _act(dtype)
+    C = 2 * G * d + H * dv
+    qkv = torch.randn(n, C + 3, generator=g).to(act)
+    ba = torch.randn(n, 2 * H + 1, generator=g).to(act)
+    rate = torch.rand(H, generator=g) * 0.5
+    bias = torch.randn(H, generator=g)
+    rows = qkv.double()
+    q = oracle.unit(rows[:, :G * d].reshape(n, G, d)) * d ** -0.5
+    k = oracle.unit(rows[:, G * d: 2 * G * d].reshape(n, G, d))
+    v = rows[:, 2 * G * d: C].reshape(n, H, dv)
+    beta = torch.sigmoid(ba.double()[:, :H])
+    dec = torch.exp(-rate.double() * oracle.softplus(
+        ba.double()[:, H + 1:] + bias.double()))
+    want = torch.zeros(n, H, dv, dtype=torch.float64)
+    for hd in range(H):
+        S = torch.zeros(d, dv, dtype=torch.float64)
+        kh = hd // (H // G)
+        for i in range(n):
+            S = dec[i, hd] * S
+            u = beta[i, hd] * (v[i, hd] - S.T @ k[i, kh])
+            S = S + torch.outer(k[i, kh], u)
+            want[i, hd] = S.T @ q[i, kh]
+    state = torch.full((3, H, dv, d), -700.0, device=device)
+    got, at = [], 0
+    for c in cuts:
+        pad = lambda t: torch.cat([t[at: at + c], torch.ones(
+            2, t.shape[1], dtype=t.dtype)]).to(device)
+        pos, _, cu, slots = _maps([c, 2], [at, -1], device, [1, 0])
+        if c == 1:            # steps of one row per sequence
+            pad = lambda t: torch.cat([t[at: at + 1], torch.ones(
+                1, t.shape[1], dtype=t.dtype)]).to(device)
+            pos, _, cu, slots = _maps([1, 1], [at, -1], device, [1, 0])
+        qq, bb = pad(qkv), pad(ba)
+        y = torch.full((qq.shape[0], H * dv), 5.0, device=device)
+        ops.delta_scan(y, qq, 0, G * d, 2 * G * d, bb, 0, H + 1,
+                       rate.to(device), bias.to(device), d ** -0.5, state,
+                       pos, cu, slots, H, G, d, dv)
+        assert float(y[c:].abs().max()) == 0.0
+        got.append(y[:c])
+        at += c
+    assert float(state[0].min()) == -700.0 and float(state[2].min()) == -700.0
+    _close(torch.cat(got), want.view(n, H * dv), dtype, f"delta {d} {dv}")
+
+
+def case_op_selective(device, dtype, I=9, N=5, cuts=(4, 1, 9, 1, 1)):
+    """The selective scan over portions with a dirty slot and an inactive
+    neighbour."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(9 + N)
+    n = sum(cuts)
+    act = _act(dtype)
+    x = torch.randn(n, I, generator=g).to(act)
+    z = torch.randn(n, I + 3, generator=g).to(act)
+    dt = torch.randn(n, I, generator=g)
+    bc = torch.randn(n, 2 * N + 2, generator=g).to(act)
+    bias = torch.randn(I, generator=g) - 1.0
+    A = -torch.exp(torch.randn(I, N, generator=g) * 0.7)
+    D = torch.randn(I, generator=g)
+    step = oracle.softplus(dt.double() + bias.double())
+    B, C = bc.double()[:, 1: 1 + N], bc.double()[:, 2 + N:]
+    S = torch.zeros(I, N, dtype=torch.float64)
+    want = torch.zeros(n, I, dtype=torch.float64)
+    for i in range(n):
+        S = torch.exp(step[i][:, None] * A.double()) * S + \
+            (step[i] * x[i].double())[:, None] * B[i][None]
+        want[i] = S @ C[i] + D.double() * x[i].double()
+    want = want * oracle.silu(z.double()[:, 3:])
+    state = torch.full((3, I, N), -700.0, device=device)
+    A2 = (A.double() / math.log(2.0)).float().to(device)
+    got, at = [], 0
+    for c in cuts:
+        k = 1 if c == 1 else 2
+        pad = lambda t: torch.cat([t[at: at + c], torch.ones(
+            k, t.shape[1], dtype=t.dtype)]).to(device)
+        pos, _, cu, slots = _maps([c, k], [at, -1], device, [1, 0])
+        xx = pad(x)
+        out = torch.full(xx.shape, 5.0, dtype=act, device=device)
+        ops.selective_scan(out, xx, pad(z)[:, 3:], pad(dt), bias.to(device),
+                           pad(bc), 1, 2 + N, A2, D.to(device), state, pos,
+                           cu, slots)
+        assert float(out[c:].abs().max()) == 0.0
+        got.append(out[:c])
+        at += c
+    assert float(state[0].min()) == -700.0 and float(state[2].min()) == -700.0
+    _close(torch.cat(got), want, dtype, f"selective {I} {N}")
+
+
+def case_op_attention(device, dtype, d=8, BS=4, n=90, start=0):
+    """The attention kernels with every option on and off against dense
+    scores: unnormed keys, the logarithmic bias, the linear one, cap, chunk,
+    window, sink, values of their own. One query and key pair per head is
+    scaled up so that its score stands out."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(11 + d)
+    H, G = 6, 2
+    act = _act(dtype)
+    nb = -(-n // BS)
+    perm = torch.randperm(nb, generator=g)
+    k = torch.randn(n, G, d, generator=g).to(act)
+    v = torch.randn(n, G, d, generator=g).to(act)
+    q = torch.randn(n - start, H * d, generator=g).to(act)
+    q[-1] = (k[n - 20].repeat_interleave(H // G, 0).reshape(-1) * 2).to(act)
+    kc = torch.full((nb, G, BS, d), 300.0, dtype=act)
+    vc = torch.full((nb, G, BS, d), 300.0, dtype=act)
+    for j in range(n):
+        kc[perm[j // BS], :, j % BS] = k[j]
+        vc[perm[j // BS], :, j % BS] = v[j]
+    r1, r2 = torch.rand(H, generator=g) + 0.3, torch.rand(H, generator=g) * 3
+    slopes = torch.rand(H, generator=g) * 0.05
+    pos, row_seq, _, _ = _maps([n - start], [start], device, [0])
+    bt = perm.to(torch.int32)[None].to(device).contiguous()
+    dd = lambda t: t.to(device)
+    full = dict(scale=1.5 * d ** -0.5, softcap=4.0, chunk=37, window=0,
+                sink=True, key_eps=1e-5, lin=False, log=True, own=False)
+    variants = [full, dict(full, sink=False), dict(full, softcap=0.0),
+                dict(full, chunk=0), dict(full, log=False),
+                dict(full, key_eps=-1.0), dict(full, chunk=0, window=33),
+                dict(full, lin=True, log=False, own=True),
+                dict(full, scale=-6.0, chunk=0)]
+    for o in variants:
+        kk = k.double()
+        if o["key_eps"] >= 0:
+            kk = oracle.unit_rms(kk, o["key_eps"])
+        vv = v.double() if o["own"] else k.double()
+        want = torch.zeros(n - start, H, d, dtype=torch.float64)
+        for i in range(start, n):
+            lo = i // o["chunk"] * o["chunk"] if o["chunk"] else 0
+            if o["window"]:
+                lo = max(lo, i - o["window"] + 1)
+            dist = (i - torch.arange(lo, i + 1)).double()
+            for h in range(H):
+                s = kk[lo: i + 1, h // (H // G)] @ \
+                    q[i - start].double().view(H, d)[h] * o["scale"]
+                if o["softcap"]:
+                    s = o["softcap"] * torch.tanh(s / o["softcap"])
+                if o["lin"]:
+                    s = s - slopes[h].double() * dist
+                if o["log"]:
+                    s = s - r1[h].double() * torch.log1p(r2[h].double() *
+                                                         dist)
+                m = max(float(s.max()), 0.0) if o["sink"] else float(s.max())
+                e = torch.exp(s - m)
+                den = e.sum() + (math.exp(-m) if o["sink"] else 0.0)
+                want[i - start, h] = (e / den) @ vv[lo: i + 1, h // (H // G)]
+        want = want.view(n - start, H * d)
+        out = torch.full((n - start, H * d), 9.0, dtype=act, device=device)
+        ops.masked_attention(
+            out, dd(q), dd(kc), dd(vc) if o["own"] else None,
+            dd(slopes) if o["lin"] else None, dd(r1) if o["log"] else None,
+            dd(r2) if o["log"] else None, pos, row_seq, bt, H, o["scale"],
+            o["softcap"], o["chunk"], o["window"], o["sink"], o["key_eps"])
+        _close(out, want, dtype, f"rows {o}")
+        if o["window"] or o["lin"] or o["own"] or \
+                not ops.masked_tiles_supported(dd(q), d, BS):
+            continue
+        i32 = lambda t: torch.tensor(t, dtype=torch.int32, device=device)
+        qb = list(range(0, n - start, 32))
+        out = torch.full((n - start, H * d), 9.0, dtype=act, device=device)
+        ops.masked_attention_tiles(
+            out, dd(q), dd(kc), dd(r1) if o["log"] else None,
+            dd(r2) if o["log"] else None, bt, i32([n]), i32([[start, 0]]),
+            i32([0] * len(qb)), i32(qb), o["scale"], o["softcap"], o["chunk"],
+            o["sink"], o["key_eps"])
+        _close(out, want, dtype, f"tiles {o}")
+
+
+def case_op_head_norm(device, dtype):
+    """Per-head query norm and the page write of the unnormed keys."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(12)
+    for H, G, d, BS in ((3, 1, 6, 4), (4, 2, 24, 16), (2, 2, 128, 16),
+                        (5, 1, 40, 4)):
+        act = _act(dtype)
+        cuts, start = [7, 2, 5], [3, -1, 0]
+        T = sum(cuts)
+        C = (H + G) * d + 8
+        proj = torch.randn(T, C, generator=g).to(act)
+        w = torch.randn(d, generator=g)
+        pos, row_seq, _, _ = _maps(cuts, start, device, [0, 1, 2])
+        bt = torch.tensor([[5, 1, 3], [0, 0, 0], [2, 4, 6]],
+                          dtype=torch.int32, device=device)
+        kc = torch.full((8, G, BS, d), 7.0, dtype=act, device=device)
+        qo = torch.full((T, H * d), 7.0, dtype=act, device=device)
+        ops.head_norm_append(qo, kc, proj.to(device), G * d + 8, 0,
+                             w.to(device), 1e-4, pos, row_seq, bt)
+        q = proj[:, G * d + 8:].double().view(T, H, d)
+        want = (oracle.unit_rms(q, 1e-4) * w.double()).view(T, H * d)
+        live = pos.cpu() >= 0
+        _close(qo.cpu()[live], want[live], dtype, "queries")
+        seen = torch.full((8, G, BS, d), 7.0, dtype=act)
+        for r in range(T):
+            p = int(pos[r])
+            if p >= 0:
+                seen[int(bt[int(row_seq[r]), p // BS]), :, p % BS] = \
+                    proj[r, :G * d].view(G, d)
+        assert torch.equal(kc.cpu(), seen)
+
+
+def case_op_router(device):
+    """Sigmoid scores as they are, ties, wider rows than needed, a NaN."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(8)
+    for E, top in ((8, 3), (6, 1), (4, 4), (17, 2)):
+        z = torch.randn(70, E, generator=g)
+        z[3] = 0.25                      # all equal: the lowest indices win
+        z[7, E - 1] = z[7].max()         # a tie between two experts
+        idx = torch.full((70, top + 1), -5, dtype=torch.int32, device=device)
+        wts = torch.zeros(70, top + 1, device=device)
+        ops.router_sigmoid(idx, wts, z.to(device), top, 1.5)
+        pick, w = oracle.route(z.double(), {"x.router": torch.eye(
+            E, dtype=torch.float64)}, "x.", {"top": top})
+        assert torch.equal(idx[:, :top].cpu().long(), pick)
+        assert int(idx[:, top].max()) == -5
+        _close(wts[:, :top], w * 1.5, "fp32", f"weights {E}")
+
+
+def case_op_experts(device, dtype):
+    """The pair kernels: weights on inputs and on outputs, clamped and plain
+    gates, an extra row, more than 32 rows of one expert, more pairs than one
+    list holds, rows off the matrix-core sizes."""
+    from kukeon_amd import ops
+    g = torch.Generator().manual_seed(14)
+    act = _act(dtype)
+    for T, E, top, W, ff in ((5, 4, 2, 24, 16), (40, 3, 3, 136, 40),
+                             (9, 5, 1, 22, 9), (70, 2, 1, 64, 72),
+                             (700, 3, 3, 16, 8)):
+        up = (ff + 7) // 8 * 8
+        h = torch.randn(T, W, generator=g).to(act)
+        gu = torch.zeros(E, 2 * up, W)
+        gu[:, :ff] = torch.randn(E, ff, W, generator=g) * W ** -0.5
+        gu[:, up: up + ff] = torch.randn(E, ff, W, generator=g) * W ** -0.5
+        dn = torch.randn(E, W, ff, generator=g) * ff ** -0.5
+        gu, dn = gu.to(act), dn.to(act)
+        idx = torch.stack([torch.randperm(E, generator=g)[:top]
+                           for _ in range(T)]).to(torch.int32)
+        wts = torch.rand(T, top, generator=g)
+        ex = torch.randn(T, W, generator=g).to(act)
+        for lim, al, sh, win, extra in ((float("inf"), 1.0, 0.0, True, None),
+                                        (0.7, 1.7, 1.0, False, ex),
+                                        (float("inf"), 1.0, 0.0, False, ex)):
+            want = torch.zeros(T, W, dtype=torch.float64)
+            for k in range(top):
+                e = idx[:, k].long()
+                z = torch.bmm(gu.double()[e], h.double()[..., None])[..., 0]
+                wk = wts[:, k].double()[:, None]
+                a, b = z[:, :ff], z[:, up: up + ff]
+                if win:
+                    a, b = a * wk, b * wk
+                a, b = a.clamp(max=lim), b.clamp(-lim, lim)
+                y = a * torch.sigmoid(al * a) * (b + sh)
+                y = torch.bmm(dn.double()[e], y[..., None])[..., 0]
+                want += y if win else wk * y
+            if extra is not None:
+                want = want + extra.double()
+            out = torch.full((T, W), 9.0, dtype=act, device=device)
+            ops.routed_experts(out, h.to(device), idx.to(device),
+                               wts.to(device), top, gu.to(device),
+                               dn.to(device), lim, al, sh, win,
+                               None if extra is None else extra.to(device))
+            _close(out, want, dtype, f"experts {T} {E} {W} {ff} {win}")
+
+
+# ------------------------------------------------- folders, programs, servers
+def case_registry(tmp_path, device, dtype):
+    """A checkpoint folder is found by its architecture name and read."""
+    from dumovik_cases import write_checkpoint
+    from kukeon_amd.models.registry import load_checkpoint
+    cfg = CONFIGS["extreme"]()
+    W = weights(cfg, 11)
+    write_checkpoint(tmp_path, cfg, W)
+    mcfg, model = load_checkpoint(str(tmp_path), device=device, dtype=dtype)
+    assert mcfg.family == "noridra" and len(model.layers) == 2
+    eng = LLMEngine(model, mcfg, EngineConfig(
+        block_size=4, max_model_len=64, max_sessions=2, state_slots=2,
+        num_kv_blocks=16, use_graphs=False), device=device)
+    toks = tokens(cfg, 13, 11)
+    got = run_schedule(eng, [toks], [[(0, 6)], [(0, 7)]])[0]
+    check(got, logits_of(cfg, W, toks), dtype, "from a folder")
+
+
+def case_trace_runner(tmp_path, device, dtype):
+    """The trace runner as a program: a checkpoint folder, steps on standard
+    input, logits files and `done` lines back. Three requests through a pool
+    sized for two, portions beside single tokens, a request left out of a
+    step."""
+    import json
+    import os
+    import subprocess
+    import sys
+    import numpy as np
+    from dumovik_cases import write_checkpoint
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 14)
+    model_dir, out_dir = tmp_path / "model", tmp_path / "out"
+    model_dir.mkdir()
+    write_checkpoint(model_dir, cfg, W)
+    prompts = {"a": tokens(cfg, 70, 90), "b": tokens(cfg, 40, 91),
+               "c": tokens(cfg, 33, 92)}
+    want = {k: logits_of(cfg, W, p) for k, p in prompts.items()}
+    steps = [[("a", 30), ("b", 1)], [("a", 1), ("b", 38)], [("a", 39)],
+             [("b", 1), ("c", 2)], [("c", 30)], [("c", 1)]]
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    cmd = [sys.executable, os.path.join(root, "bin", "trace_run"), "--model",
+           str(model_dir), "--dtype",
+           "float32" if dtype == "fp32" else "bfloat16", "--out",
+           str(out_dir), "--max-tokens", "128", "--slots", "2", "--device",
+           device]
+    p = subprocess.Popen(cmd, stdin=subprocess.PIPE, stdout=subprocess.PIPE,
+                         text=True, cwd=root)
+    at = {k: 0 for k in prompts}
+    try:
+        for n, step in enumerate(steps):
+            entries, end = [], []
+            for k, cnt in step:
+                toks = prompts[k][at[k]: at[k] + cnt]
+                entries.append({"id": k, "tokens": toks,
+                                "want": [0, cnt - 1] if cnt > 1 else [0]})
+                at[k] += cnt
+                if at[k] == len(prompts[k]):
+                    end.append(k)
+            p.stdin.write(json.dumps({"step": n, "entries": entries,
+                                      "end": end}) + "\n")
+            p.stdin.flush()
+            line = p.stdout.readline()
+            while line and line.strip() != "done %d" % n:
+                line = p.stdout.readline()
+            assert line, "the runner ended early"
+            got = torch.from_numpy(np.fromfile(
+                out_dir / ("%d.f32" % n), dtype="<f4").reshape(
+                -1, cfg["vocab"]))
+            rows = [want[k][at[k] - cnt + w] for k, cnt in step
+                    for w in ([0, cnt - 1] if cnt > 1 else [0])]
+            assert len(rows) == got.shape[0]
+            check(got, torch.stack(rows), dtype, f"step {n}")
+        p.stdin.close()
+        assert p.wait(timeout=60) == 0
+    finally:
+        if p.poll() is None:
+            p.kill()
+
+
+def case_modelhub(device):
+    """The serving daemon's model server with this family: sessions over the
+    unix socket, two turns on one session, greedy tokens as the plain model
+    gives them."""
+    import uuid
+    from kukeon_amd.serve.server import ModelhubClient, ModelhubServer
+    cfg = CONFIGS["hybrid"]()
+    W = weights(cfg, 16)
+    mcfg = NoridraConfig.from_json(cfg)
+    model = NoridraModel(mcfg, device=device, dtype="fp32", tensors=W,
+                         max_position=128)
+    ecfg = EngineConfig(block_size=4, max_model_len=128, max_sessions=4,
+                        state_slots=4, num_kv_blocks=64, use_graphs=False)
+    sock = f"/tmp/mh-{uuid.uuid4().hex[:10]}.sock"
+    hub = ModelhubServer(model, mcfg, ecfg, sock, device=device)
+    hub.start()
+    try:
+        c = ModelhubClient(sock, timeout=120)
+        p1, p2 = tokens(cfg, 6, 70), tokens(cfg, 3, 71)
+        r1 = c.generate("s", p1, max_new_tokens=4, temperature=0.0)
+        assert len(r1["tokens"]) == 4
+        assert_greedy(cfg, W, p1, r1["tokens"], "first turn")
+        r2 = c.generate("s", p2, max_new_tokens=3, temperature=0.0)
+        assert len(r2["tokens"]) == 3
+        assert_greedy(cfg, W, p1 + r1["tokens"] + p2, r2["tokens"],
+                      "second turn")
+        rb = c.generate("t", p2, max_new_tokens=2, temperature=0.0)
+        assert_greedy(cfg, W, p2, rb["tokens"], "other session")
+        assert c.call("stats")["sessions"] == 2
+        c.close()
+    finally:
+        hub.stop()
+
+
+def case_real_sizes(device, say=lambda s: None):
+    """A stack at the layer sizes of a served model (heads of 128, pages of
+    16, rows of thousands of entries): the bf16 serving kernels against the
+    exact fp32 kernels, prompts on the packed path and decoding under
+    hipGraphs."""
+    from kukeon_amd.models.noridra import noridra_bench, random_tensors
+    mcfg = noridra_bench(width=2048, layers=4, heads=16, kv_heads=4, ff=4096,
+                         vocab=512, chunk=96, experts=16, max_positions=512,
+                         name="noridra-sizes")
+    W = random_tensors(mcfg, 5)
+    g = torch.Generator().manual_seed(9)
+    prompts = [torch.randint(0, 512, (n,), generator=g).tolist()
+               for n in (150, 70, 129)]
+    outs = {}
+    for dtype in ("fp32", "bf16"):
+        say(f"model {dtype}")
+        model = NoridraModel(mcfg, device=device, dtype=dtype, tensors=W)
+        eng = LLMEngine(model, mcfg, EngineConfig(
+            block_size=16, max_model_len=512, max_sessions=4, state_slots=4,
+            num_kv_blocks=64, use_graphs=False), device=device)
+        say("prompts")
+        kvs = [SequenceKV(16) for _ in prompts]
+        lg = [eng.forward_tokens([(kv, p[:-6]) for kv, p in
+                                  zip(kvs, prompts)])]
+        say("single tokens")
+        for k in range(6, 0, -1):
+            lg.append(eng.forward_tokens([(kv, [p[-k]]) for kv, p in
+                                          zip(kvs, prompts)]))
+        outs[dtype] = torch.cat(lg).float().cpu()
+        assert bool(torch.isfinite(outs[dtype]).all())
+        for kv in kvs:
+            eng.free_sequence(kv)
+        if dtype == "bf16":
+            say("generation under graphs")
+            eng.ecfg.use_graphs = True
+            eng.ecfg.graph_buckets = (4,)
+            eng.ecfg.decode_microbatch = 8
+            sp = SamplingParams(temperature=0.7, top_k=50, top_p=0.9,
+                                max_new_tokens=17)
+            kvs = [SequenceKV(16) for _ in prompts]
+            rids = [eng.add_request(kv, p, sp) for kv, p in
+                    zip(kvs, prompts)]
+            n = 0
+            while eng.has_work():
+                for o in eng.step():
+                    n += len(o.new_tokens)
+                    assert all(0 <= t < 512 for t in o.new_tokens)
+            assert n == 17 * len(rids)
+        del eng, model
+    e = row_errors(outs["bf16"], outs["fp32"])
+    over = int((e > 0.15).sum())
+    assert over <= max(1, e.numel() // 4), f"{over} rows off, worst " \
+        f"{float(e.max()):.3g}"
