@@ -31,8 +31,8 @@ COMPARE_SIZES = {
 
 
 def compare_families(args) -> None:
-    """Prefill and decode tokens/s of Lipedra, Rasesun, Dumovik or Bezizen
-    and of Llama (or another family) through the same engine at equal sizes: same
+    """Prefill and decode tokens/s of Lipedra, Rasesun, Dumovik, Bezizen or
+    Noridra and of Llama (or another family) through the same engine at equal sizes: same
     width, head counts,
     feed-forward size, layer count and vocabulary (Llama head_dim 128;
     Lipedra two score maps of 64 and value rows of 128 — equal cache bytes
@@ -44,7 +44,9 @@ def compare_families(args) -> None:
     active; Bezizen four residual streams, three wkv layers to one parallel
     layer of windowed attention over 1024 tokens beside a gated linear
     attention, a shared expert everywhere and every second feed-forward a
-    mixture of 16 routed experts, two active)."""
+    mixture of 16 routed experts, two active; Noridra delta rule, attention
+    over 8192-token chunks, selective scan and delta rule, every second
+    feed-forward a mixture of 16 routed experts, two active)."""
     from kukeon_amd.engine.config import (EngineConfig, ModelConfig,
                                           SamplingParams)
     from kukeon_amd.engine.engine import LLMEngine
@@ -53,6 +55,7 @@ def compare_families(args) -> None:
     from kukeon_amd.models.bezizen import bezizen_bench
     from kukeon_amd.models.dumovik import dumovik_bench
     from kukeon_amd.models.lipedra import lipedra_bench
+    from kukeon_amd.models.noridra import noridra_bench
     from kukeon_amd.models.rasesun import rasesun_bench
 
     device = args.device or ("cuda:0" if torch.cuda.is_available() else "cpu")
@@ -84,6 +87,13 @@ def compare_families(args) -> None:
                                     experts=16 if on_gpu else 4,
                                     max_positions=2048,
                                     name=f"bezizen-{size}")
+            elif fam == "noridra":
+                cfg = noridra_bench(width=W, layers=nl, heads=hq,
+                                    kv_heads=hk, ff=ff, vocab=vocab,
+                                    chunk=8192 if on_gpu else 16,
+                                    experts=16 if on_gpu else 4,
+                                    max_positions=2048,
+                                    name=f"noridra-{size}")
             elif fam == "dumovik":
                 cfg = dumovik_bench(width=W, layers=nl, heads=hq,
                                     kv_heads=hk, ff=ff, vocab=vocab,
@@ -177,11 +187,13 @@ def main() -> None:
                          "decode throughput of the Lipedra family beside "
                          "Llama at equal layer sizes (random weights)")
     ap.add_argument("--compare-family", default="lipedra",
-                    choices=["lipedra", "rasesun", "dumovik", "bezizen"],
+                    choices=["lipedra", "rasesun", "dumovik", "bezizen",
+                             "noridra"],
                     help="with --compare-families: the family that runs "
                          "beside Llama")
     ap.add_argument("--compare-against", default="llama",
-                    choices=["llama", "lipedra", "rasesun", "dumovik"],
+                    choices=["llama", "lipedra", "rasesun", "dumovik",
+                             "bezizen"],
                     help="with --compare-families: the family it runs "
                          "beside (default Llama)")
     ap.add_argument("--compare-sizes", default="2k,4k,8k",

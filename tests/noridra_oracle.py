@@ -154,11 +154,20 @@ MIXERS = {"delta": delta_mixer, "attention": attention_mixer,
 
 
 # ---- mixture of experts -----------------------------------------------------
-def route(h, t, p, r):
-    """-> (chosen experts [T, top], their weights [T, top])."""
+def route(h, t, p, r, given=None):
+    """-> (chosen experts [T, top], their weights [T, top]). `given` is a
+    choice made elsewhere on rounded numbers: it is taken over where its
+    scores are within a small distance of the best ones (a close call), so
+    that both sides go on with the same experts."""
+    top = int(r["top"])
     s = torch.sigmoid(lin(h, t[p + "router"]))
     pick = torch.sort(s, dim=-1, descending=True,
-                      stable=True).indices[:, :int(r["top"])]
+                      stable=True).indices[:, :top]
+    if given is not None:
+        assert all(len(set(row.tolist())) == top for row in given)
+        best, theirs = s.gather(1, pick), s.gather(1, given)
+        close = (best.min(-1).values - theirs.min(-1).values) < 0.1
+        pick = torch.where(close[:, None], given, pick)
     return pick, s.gather(1, pick)
 
 
@@ -167,8 +176,8 @@ def expert(h, t, p):
                t[p + "down"])
 
 
-def moe(h, t, p, f):
-    pick, w = route(h, t, p, f["router"])
+def moe(h, t, p, f, given=None):
+    pick, w = route(h, t, p, f["router"], given)
     out = torch.zeros_like(h)
     for i in range(h.shape[0]):
         for e, we in zip(pick[i].tolist(), w[i]):
@@ -177,9 +186,11 @@ def moe(h, t, p, f):
 
 
 # ---- the whole model --------------------------------------------------------
-def forward(tokens, tensors, cfg, taps=None):
+def forward(tokens, tensors, cfg, taps=None, choices=None):
     """-> logits [T, vocab]; `taps`, if a list, receives the residual stream
-    after every layer."""
+    after every layer. `choices`: per layer with a feed-forward, experts
+    chosen elsewhere [T, top] (see route)."""
+    choices = list(choices) if choices is not None else None
     t = {k: v.to(F64) for k, v in tensors.items()}
     eps = float(cfg["norm"]["eps"])
     alpha = float(cfg["postln_alpha"])
@@ -190,7 +201,8 @@ def forward(tokens, tensors, cfg, taps=None):
                               L["mixer"], eps)
         x = group_norm(alpha * x + t[p + "ls1"] * y, t[p + "norm1"], cfg)
         if L.get("mlp"):
-            y = moe(canon(x, t[p + "canon2"]), t, p + "mlp.", L["mlp"])
+            y = moe(canon(x, t[p + "canon2"]), t, p + "mlp.", L["mlp"],
+                    choices.pop(0) if choices is not None else None)
             x = group_norm(alpha * x + t[p + "ls2"] * y, t[p + "norm2"], cfg)
         if taps is not None:
             taps.append(x)
