@@ -135,7 +135,7 @@ DEV_INLINE unsigned int cvt_pk_bf16(float lo, float hi) {
 // square (formed while the tile is staged), and a sink: the softmax starts from
 // a score of 0 that has no value.
 template <int BS, bool FP8, int EXT>
-__global__ __launch_bounds__(256, 1) void prefill_attn_kernel(
+__global__ __launch_bounds__(256, EXT == 2 ? 2 : 1) void prefill_attn_kernel(
     unsigned short* __restrict__ out,       // [T, Hq*D]
     const unsigned short* __restrict__ q,   // [T, q_stride] fused qkv rows
     const void* __restrict__ k_cache,       // [NB, Hk, BS, D] bf16|fp8

@@ -34,117 +34,138 @@ DEV_INLINE float re_glu(float g, float u, const GluForm f) {
   return g / (1.0f + expf(-f.alpha * g)) * (u + f.shift);
 }
 
-#define RE_MAX_PAIRS 2048
 #define RE_ROWS 8               // output rows per wave, pair-major form
+#define RE_LIST 1024            // pairs of one expert listed at a time
 
-// this workgroup's pairs among [base, base + count): their numbers go to list
-DEV_INLINE int re_list(int* list, int* count, const int* __restrict__ idx,
-                       int ldi, int top, int base, int num, int e) {
-  __syncthreads();
-  if (threadIdx.x == 0) *count = 0;
-  __syncthreads();
-  for (int i = threadIdx.x; i < num; i += blockDim.x) {
-    const int pair = base + i;
-    if (idx[(long)(pair / top) * ldi + pair % top] == e)
-      list[atomicAdd(count, 1)] = pair;
+// The pairs among [from, pairs) routed to expert e, in order, up to RE_LIST of
+// them, by one wave into its own list; `from` moves to the first pair not
+// looked at. -> how many.
+DEV_INLINE int re_list(int* list, const int* __restrict__ idx, int ldi, int top,
+                       int pairs, int e, int& from) {
+  const int lane = threadIdx.x & (WAVE - 1);
+  int n = 0;
+  while (from < pairs && n + WAVE <= RE_LIST) {
+    const int pair = from + lane;
+    const bool mine = pair < pairs &&
+                      idx[(long)(pair / top) * ldi + pair % top] == e;
+    const unsigned long long m = __ballot(mine);
+    if (mine) list[n + __popcll(m & ((1ull << lane) - 1ull))] = pair;
+    n += __popcll(m);
+    from += WAVE;
   }
-  __syncthreads();
-  return *count;
+  __builtin_amdgcn_wave_barrier();       // wave-private LDS, in order
+  return n;
 }
 
-// One wave: 16 weight rows of wa (and of wb when UP) against up to 32 listed
-// pairs at a time, v_mfma_f32_16x16x32_bf16 with the weights as A (lane = row,
-// 8 consecutive k) and the pairs' rows as B. A lane fetches 64 contiguous bytes
-// per 128 entries of k; the same permutation of k on both operands leaves the
-// product unchanged. Output lane (pair = l & 15) holds rows 4 (l >> 4) + r.
+// A workgroup owns 16 gate rows and the 16 up rows beside them (UP), or 32 rows
+// of W_down, of one expert. Its four waves share out the reduction in blocks of
+// 128 entries (wave w takes blocks w, w + 4, ...), so a weight row is read once
+// and an input row once per workgroup; v_mfma_f32_16x16x32_bf16 with the
+// weights as A (lane = row, 8 consecutive k) and up to 32 listed pairs' rows as
+// B; the waves' sums meet in LDS, added in wave order. Output lane (pair = l &
+// 15) holds rows 4 (l >> 4) + r.
 template <bool UP>
 __global__ __launch_bounds__(256) void routed_mfma_kernel(
     void* __restrict__ dst, const bf16_t* __restrict__ src,
     const int* __restrict__ idx, int ldi, const float* __restrict__ wts, int ldw,
     const bf16_t* __restrict__ w, int NR, int wrows, int up_row, int K, int top,
     int pairs, int weigh, GluForm form) {
-  __shared__ int list[RE_MAX_PAIRS];
-  __shared__ int count;
+  __shared__ int lists[4][RE_LIST];
+  __shared__ float sums[4][2][2][16 * 17];   // [wave][rows][pairs][pair, row]
   const int e = blockIdx.x;
   const int lane = threadIdx.x & (WAVE - 1);
   const int wave = threadIdx.x / WAVE;
   const int rc = lane & 15;
   const int g4 = lane >> 4;
-  const int r0 = (blockIdx.y * 4 + wave) * 16;
-  const int arow = min(r0 + rc, NR - 1);
-  const bf16_t* wa = w + ((long)e * wrows + arow) * K + g4 * 32;
-  const bf16_t* wb = wa + (long)up_row * K;
+  int* list = lists[wave];
+  const int r0 = blockIdx.y * (UP ? 16 : 32);
+  const int row0 = min(r0 + rc, NR - 1);
+  const int row1 = UP ? up_row + row0 : min(r0 + 16 + rc, NR - 1);
+  const bf16_t* wa = w + ((long)e * wrows + row0) * K + g4 * 8;
+  const bf16_t* wb = w + ((long)e * wrows + row1) * K + g4 * 8;
   const uint4 zero = uint4{0u, 0u, 0u, 0u};
-  for (int base = 0; base < pairs; base += RE_MAX_PAIRS) {
-    const int n = re_list(list, &count, idx, ldi, top, base,
-                          min(RE_MAX_PAIRS, pairs - base), e);
-    if (r0 >= NR) continue;              // no barrier below this point
+  int from = 0;
+  while (from < pairs) {
+    const int n = re_list(list, idx, ldi, top, pairs, e, from);
     for (int g0 = 0; g0 < n; g0 += 32) {
       const bool two = g0 + 16 < n;
-      int pair[2];
-      const bf16_t* xr[2];
-#pragma unroll
-      for (int q = 0; q < 2; ++q) {
-        const int i = g0 + q * 16 + rc;
-        pair[q] = i < n ? list[i] : -1;
-        const int sr = pair[q] < 0 ? 0 : (UP ? pair[q] / top : pair[q]);
-        xr[q] = src + (long)sr * K + g4 * 32;
-      }
-      re_f32x4_v aa[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-      re_f32x4_v bb[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+      const int p0 = g0 + rc < n ? list[g0 + rc] : -1;
+      const int p1 = g0 + 16 + rc < n ? list[g0 + 16 + rc] : -1;
+      const bf16_t* x0 =
+          src + (long)(p0 < 0 ? 0 : (UP ? p0 / top : p0)) * K + g4 * 8;
+      const bf16_t* x1 =
+          src + (long)(p1 < 0 ? 0 : (UP ? p1 / top : p1)) * K + g4 * 8;
+      re_f32x4_v acc[2][2] = {{{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}},
+                              {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}}};
 #pragma unroll 2
-      for (int k0 = 0; k0 < K; k0 += 128) {
-        uint4 a[4], b[4], x[2][4];
+      for (int k0 = wave * 128; k0 < K; k0 += 512) {
+        uint4 a[4], b[4], x[4], z[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const bool in = k0 + g4 * 32 + i * 8 < K;
-          a[i] = in ? *reinterpret_cast<const uint4*>(wa + k0 + i * 8) : zero;
-          if (UP)
-            b[i] = in ? *reinterpret_cast<const uint4*>(wb + k0 + i * 8) : zero;
-          x[0][i] = in && pair[0] >= 0
-                        ? *reinterpret_cast<const uint4*>(xr[0] + k0 + i * 8)
-                        : zero;
-          x[1][i] = two && in && pair[1] >= 0
-                        ? *reinterpret_cast<const uint4*>(xr[1] + k0 + i * 8)
-                        : zero;
-        }
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          aa[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              re_frag(a[i]), re_frag(x[0][i]), aa[0], 0, 0, 0);
-          if (UP)
-            bb[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                re_frag(b[i]), re_frag(x[0][i]), bb[0], 0, 0, 0);
+          const int k = k0 + i * 32;
+          const bool in = k + g4 * 8 < K;
+          a[i] = in ? *reinterpret_cast<const uint4*>(wa + k) : zero;
+          b[i] = in ? *reinterpret_cast<const uint4*>(wb + k) : zero;
+          x[i] = in && p0 >= 0 ? *reinterpret_cast<const uint4*>(x0 + k) : zero;
+          z[i] = zero;
         }
         if (two) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            aa[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                re_frag(a[i]), re_frag(x[1][i]), aa[1], 0, 0, 0);
-            if (UP)
-              bb[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                  re_frag(b[i]), re_frag(x[1][i]), bb[1], 0, 0, 0);
+            const int k = k0 + i * 32;
+            if (k + g4 * 8 < K && p1 >= 0)
+              z[i] = *reinterpret_cast<const uint4*>(x1 + k);
+          }
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          acc[0][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              re_frag(a[i]), re_frag(x[i]), acc[0][0], 0, 0, 0);
+          acc[1][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              re_frag(b[i]), re_frag(x[i]), acc[1][0], 0, 0, 0);
+        }
+        if (two) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            acc[0][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                re_frag(a[i]), re_frag(z[i]), acc[0][1], 0, 0, 0);
+            acc[1][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                re_frag(b[i]), re_frag(z[i]), acc[1][1], 0, 0, 0);
           }
         }
       }
+      __syncthreads();                   // the previous sums are read
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int q = 0; q < 2; ++q)
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            sums[wave][h][q][rc * 17 + 4 * g4 + r] = acc[h][q][r];
+      __syncthreads();
+      // thread -> (pair of the 32, row of the 16), two pairs per thread
 #pragma unroll
       for (int q = 0; q < 2; ++q) {
-        if (pair[q] < 0) continue;
-        const float s =
-            UP && weigh
-                ? wts[(long)(pair[q] / top) * ldw + pair[q] % top]
-                : 1.0f;
+        const int pi = threadIdx.x >> 4, row = threadIdx.x & 15;
+        const int li = g0 + q * 16 + pi;
+        if (li >= n) continue;
+        const long pair = list[li];
+        float s0 = 0.f, s1 = 0.f;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int row = r0 + 4 * g4 + r;
-          if (row < NR) {
-            const long at = (long)pair[q] * NR + row;
-            if (UP)
-              reinterpret_cast<bf16_t*>(dst)[at] =
-                  f2us(re_glu(s * aa[q][r], s * bb[q][r], form));
-            else
-              reinterpret_cast<float*>(dst)[at] = aa[q][r];
-          }
+        for (int v = 0; v < 4; ++v) {
+          s0 += sums[v][0][q][pi * 17 + row];
+          s1 += sums[v][1][q][pi * 17 + row];
+        }
+        if (UP) {
+          const float s =
+              weigh ? wts[(pair / top) * ldw + pair % top] : 1.0f;
+          if (r0 + row < NR)
+            reinterpret_cast<bf16_t*>(dst)[pair * NR + r0 + row] =
+                f2us(re_glu(s * s0, s * s1, form));
+        } else {
+          float* o = reinterpret_cast<float*>(dst) + pair * NR + r0 + row;
+          if (r0 + row < NR) o[0] = s0;
+          if (r0 + 16 + row < NR) o[16] = s1;
         }
       }
     }
@@ -261,7 +282,7 @@ void routed_experts(torch::Tensor out, torch::Tensor h, torch::Tensor idx,
   KK_DISPATCH_ACT(h, {
     if (up_mfma)
       routed_mfma_kernel<true><<<
-          dim3((unsigned)E, (unsigned)((ff + 63) / 64)), 256, 0, stream>>>(
+          dim3((unsigned)E, (unsigned)((ff + 15) / 16)), 256, 0, stream>>>(
           act.data_ptr(), reinterpret_cast<const bf16_t*>(h.data_ptr()),
           idx.data_ptr<int>(), ldi, wts.data_ptr<float>(), ldw,
           reinterpret_cast<const bf16_t*>(w_gu.data_ptr()), ff, wrows, up_row,
@@ -276,7 +297,7 @@ void routed_experts(torch::Tensor out, torch::Tensor h, torch::Tensor idx,
           (int)top, (int)weigh_input, form);
     if (down_mfma)
       routed_mfma_kernel<false><<<
-          dim3((unsigned)E, (unsigned)((W + 63) / 64)), 256, 0, stream>>>(
+          dim3((unsigned)E, (unsigned)((W + 31) / 32)), 256, 0, stream>>>(
           part.data_ptr(), reinterpret_cast<const bf16_t*>(act.data_ptr()),
           idx.data_ptr<int>(), ldi, wts.data_ptr<float>(), ldw,
           reinterpret_cast<const bf16_t*>(w_down.data_ptr()), W, W, 0, ff,

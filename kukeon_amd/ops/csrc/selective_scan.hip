@@ -19,7 +19,16 @@
 namespace kukeon {
 
 #define SS_TT 32
-#define SS_PF 8                 // tokens fetched ahead
+
+// softplus: log1p(e) = e log(u) / (u - 1) with u = 1 + e rounded makes up for
+// the digits that 1 + e drops
+DEV_INLINE float ss_softplus(float a) {
+  if (a > 20.f) return a;
+  const float e = __expf(a);
+  const float u = 1.0f + e;
+  const float d = u - 1.0f;
+  return d == 0.f ? e : e * (__logf(u) / d);
+}
 
 template <int CTRL>
 DEV_INLINE float ss_dpp_add(float v) {
@@ -36,7 +45,9 @@ DEV_INLINE float ss_lanes_sum(float v) {
   return v;
 }
 
-template <typename T, int LN, int NR>
+// PF: tokens fetched ahead; 1 for steps of one token per sequence, whose few
+// inputs are fetched before the state (loads complete in issue order)
+template <typename T, int LN, int NR, int PF>
 __global__ __launch_bounds__(256) void selective_scan_kernel(
     T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ z,
     long ldz, const float* __restrict__ dt, long lddt,
@@ -48,8 +59,9 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
     int I, int N) {
   constexpr int NP = LN * NR;
   constexpr int NC = 256 / LN;
-  __shared__ __align__(16) float sB[SS_TT * NP];
-  __shared__ __align__(16) float sC[SS_TT * NP];
+  constexpr int TT = PF == 1 ? 1 : SS_TT;
+  __shared__ __align__(16) float sB[TT * NP];
+  __shared__ __align__(16) float sC[TT * NP];
   const int s = blockIdx.x;
   const long row0 = cu_rows[s];
   const int n = cu_rows[s + 1] - (int)row0;
@@ -64,6 +76,16 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
     if (live && l == 0)
       for (int t = 0; t < n; ++t) stf(out + (row0 + t) * (long)I + c, 0.f);
     return;
+  }
+  float px[PF], pd[PF], pz[PF], pb = 0.f, pc = 0.f;
+  if (PF == 1) {
+    px[0] = ldf(x + row0 * (long)I + cc);
+    pd[0] = dt[row0 * lddt + cc];
+    pz[0] = ldf(z + row0 * ldz + cc);
+    if (tid < N) {
+      pb = ldf(bc + row0 * ldbc + b_col + tid);
+      pc = ldf(bc + row0 * ldbc + c_col + tid);
+    }
   }
   const float bias = dt_bias[cc], skip = D[cc];
   float* st = state + ((long)state_slots[s] * I + cc) * (long)N;
@@ -92,9 +114,12 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
     S[4 * i] = sv.x; S[4 * i + 1] = sv.y; S[4 * i + 2] = sv.z; S[4 * i + 3] = sv.w;
     A[4 * i] = av.x; A[4 * i + 1] = av.y; A[4 * i + 2] = av.z; A[4 * i + 3] = av.w;
   }
-  for (int t0 = 0; t0 < n; t0 += SS_TT) {
-    const int nt = min(SS_TT, n - t0);
+  for (int t0 = 0; t0 < n; t0 += TT) {
+    const int nt = min(TT, n - t0);
     __syncthreads();
+    if (PF == 1 && t0 == 0) {
+      if (tid < NP) { sB[tid] = pb; sC[tid] = pc; }
+    } else
     for (int i = tid; i < nt * NP; i += 256) {
       const int t = i / NP, nn = i - t * NP;
       const T* row = bc + (row0 + t0 + t) * ldbc + nn;
@@ -102,12 +127,12 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
       sC[i] = nn < N ? ldf(row + c_col) : 0.f;
     }
     __syncthreads();
-    for (int t1 = 0; t1 < nt; t1 += SS_PF) {
-      const int np = min(SS_PF, nt - t1);
+    for (int t1 = 0; t1 < nt; t1 += PF) {
+      const int np = min(PF, nt - t1);
       const long r1 = row0 + t0 + t1;
-      float px[SS_PF], pd[SS_PF], pz[SS_PF];
 #pragma unroll
-      for (int k = 0; k < SS_PF; ++k) {
+      for (int k = 0; k < PF; ++k) {
+        if (PF == 1 && t0 == 0) break;
         px[k] = 0.f; pd[k] = 0.f; pz[k] = 0.f;
         if (k < np) {
           px[k] = ldf(x + (r1 + k) * (long)I + cc);
@@ -116,10 +141,10 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
         }
       }
 #pragma unroll
-      for (int k = 0; k < SS_PF; ++k) {
+      for (int k = 0; k < PF; ++k) {
         if (k >= np) break;
         const float a = pd[k] + bias;
-        const float step = a > 20.f ? a : log1pf(expf(a));
+        const float step = ss_softplus(a);
         const float dx = step * px[k];
         const float4* bt =
             reinterpret_cast<const float4*>(sB + (t1 + k) * NP) + l;
@@ -142,7 +167,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
         float yv = ss_lanes_sum<LN>((acc[0] + acc[1]) + (acc[2] + acc[3]));
         if (live && l == 0) {
           yv = fmaf(skip, px[k], yv);
-          const float g = pz[k] / (1.0f + expf(-pz[k]));
+          const float g = pz[k] / (1.0f + __expf(-pz[k]));
           stf(out + (r1 + k) * (long)I + c, yv * g);
         }
       }
@@ -202,11 +227,11 @@ void selective_scan(torch::Tensor out, torch::Tensor x, torch::Tensor z,
   if (rows == 0 || nseq == 0) return;
   TORCH_CHECK(N >= 1 && N <= 128, "selective_scan: 1 to 128 states per channel");
   auto stream = c10::hip::getCurrentHIPStream().stream();
-#define KK_LAUNCH(LN_, NR_)                                                   \
+#define KK_LAUNCH(LN_, NR_, PF_)                                                 \
   {                                                                           \
     constexpr long NC_ = 256 / LN_;                                           \
     dim3 grid((unsigned)nseq, (unsigned)((I + NC_ - 1) / NC_));               \
-    selective_scan_kernel<T, LN_, NR_><<<grid, 256, 0, stream>>>(             \
+    selective_scan_kernel<T, LN_, NR_, PF_><<<grid, 256, 0, stream>>>(             \
         reinterpret_cast<T*>(out.data_ptr()),                                 \
         reinterpret_cast<const T*>(x.data_ptr()),                             \
         reinterpret_cast<const T*>(z.data_ptr()), (long)z.stride(0),          \
@@ -219,15 +244,21 @@ void selective_scan(torch::Tensor out, torch::Tensor x, torch::Tensor z,
   }
   // one token per sequence, or too few channels to fill the device: spread a
   // channel's states over lanes; otherwise keep them in one or two threads
-  const bool spread = rows == nseq || nseq * I < 128 * 1024;
+  const bool step = rows == nseq;
+  const bool spread = nseq * I < 128 * 1024;
+#define KK_PICK(L1, N1, L2, N2)                                               \
+  if (step) KK_LAUNCH(L1, N1, 1)                                              \
+  else if (spread) KK_LAUNCH(L1, N1, 8)                                       \
+  else KK_LAUNCH(L2, N2, 8)
   KK_DISPATCH_ACT(x, {
-    if (N <= 4) KK_LAUNCH(1, 4)
-    else if (N <= 8) { if (spread) KK_LAUNCH(2, 4) else KK_LAUNCH(1, 8) }
-    else if (N <= 16) { if (spread) KK_LAUNCH(4, 4) else KK_LAUNCH(1, 16) }
-    else if (N <= 32) { if (spread) KK_LAUNCH(8, 4) else KK_LAUNCH(2, 16) }
-    else if (N <= 64) { if (spread) KK_LAUNCH(16, 4) else KK_LAUNCH(4, 16) }
-    else { if (spread) KK_LAUNCH(16, 8) else KK_LAUNCH(8, 16) }
+    if (N <= 4) { KK_PICK(1, 4, 1, 4) }
+    else if (N <= 8) { KK_PICK(2, 4, 1, 8) }
+    else if (N <= 16) { KK_PICK(4, 4, 1, 16) }
+    else if (N <= 32) { KK_PICK(8, 4, 2, 16) }
+    else if (N <= 64) { KK_PICK(16, 4, 4, 16) }
+    else { KK_PICK(16, 8, 8, 16) }
   });
+#undef KK_PICK
 #undef KK_LAUNCH
   HIP_CHECK_KERNEL();
 }

@@ -25,8 +25,28 @@ DEV_INLINE float gate_act(float g, int act) {
   return act == 0 ? g * s : s;
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void embed_streams_kernel(
+// 4 consecutive elements in the storage format
+DEV_INLINE void ld4(const float* p, float* o) {
+  const float4 a = *reinterpret_cast<const float4*>(p);
+  o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w;
+}
+DEV_INLINE void ld4(const bf16_t* p, float* o) {
+  const uint2 a = *reinterpret_cast<const uint2*>(p);
+  o[0] = us2f((unsigned short)(a.x & 0xffffu)); o[1] = us2f((unsigned short)(a.x >> 16));
+  o[2] = us2f((unsigned short)(a.y & 0xffffu)); o[3] = us2f((unsigned short)(a.y >> 16));
+}
+DEV_INLINE void st4(float* p, const float* v) {
+  *reinterpret_cast<float4*>(p) = float4{v[0], v[1], v[2], v[3]};
+}
+DEV_INLINE void st4(bf16_t* p, const float* v) {
+  *reinterpret_cast<uint2*>(p) =
+      uint2{(unsigned)f2us(v[0]) | ((unsigned)f2us(v[1]) << 16),
+            (unsigned)f2us(v[2]) | ((unsigned)f2us(v[3]) << 16)};
+}
+
+// V = 4: W is a multiple of 4 and all rows 16-byte aligned (8 for bf16)
+template <typename T, int V>
+__global__ __launch_bounds__(1024) void embed_streams_kernel(
     float* __restrict__ xs, const int* __restrict__ ids,
     const int* __restrict__ positions, const T* __restrict__ table,
     const T* __restrict__ pos_table, float scale, int S, int W, long vocab,
@@ -43,10 +63,24 @@ __global__ __launch_bounds__(256) void embed_streams_kernel(
   const T* er = table + id * (long)W;
   const T* pr = pos_table ? pos_table + (long)(p < npos ? p : npos - 1) * W
                           : nullptr;
-  for (int i = threadIdx.x; i < W; i += blockDim.x) {
-    float v = ldf(er + i) * scale;
-    if (pr) v += ldf(pr + i);
-    for (int s = 0; s < S; ++s) xr[(long)s * W + i] = v;
+  for (int i = threadIdx.x * V; i < W; i += blockDim.x * V) {
+    float v[V], q[V];
+    if (V == 4) {
+      ld4(er + i, v);
+      if (pr) ld4(pr + i, q);
+    } else {
+      v[0] = ldf(er + i);
+      if (pr) q[0] = ldf(pr + i);
+    }
+#pragma unroll
+    for (int k = 0; k < V; ++k) {
+      v[k] *= scale;
+      if (pr) v[k] += q[k];
+    }
+    for (int s = 0; s < S; ++s) {
+      if (V == 4) st4(xr + (long)s * W + i, v);
+      else xr[(long)s * W + i] = v[0];
+    }
   }
 }
 
@@ -66,34 +100,27 @@ void embed_streams(torch::Tensor xs, torch::Tensor ids, torch::Tensor positions,
                 pos_table.scalar_type() == table.scalar_type());
   if (rows == 0) return;
   auto stream = c10::hip::getCurrentHIPStream().stream();
+  const bool vec = W % 4 == 0 && aligned16(xs.data_ptr()) &&
+                   aligned16(table.data_ptr()) &&
+                   (!hp || aligned16(pos_table.data_ptr()));
+  const int want = (W / (vec ? 4 : 1) + 63) / 64 * 64;
+  const int threads = want < 64 ? 64 : (want > 1024 ? 1024 : want);
+#define KK_ARGS xs.data_ptr<float>(), ids.data_ptr<int>(),                    \
+        positions.data_ptr<int>(),                                            \
+        reinterpret_cast<const T*>(table.data_ptr()),                         \
+        hp ? reinterpret_cast<const T*>(pos_table.data_ptr()) : nullptr,      \
+        (float)scale, S, W, (long)table.size(0),                              \
+        hp ? (long)pos_table.size(0) : 0L
   KK_DISPATCH_ACT(table, {
-    embed_streams_kernel<T><<<dim3((unsigned)rows), 256, 0, stream>>>(
-        xs.data_ptr<float>(), ids.data_ptr<int>(), positions.data_ptr<int>(),
-        reinterpret_cast<const T*>(table.data_ptr()),
-        hp ? reinterpret_cast<const T*>(pos_table.data_ptr()) : nullptr,
-        (float)scale, S, W, (long)table.size(0),
-        hp ? (long)pos_table.size(0) : 0L);
+    if (vec)
+      embed_streams_kernel<T, 4><<<dim3((unsigned)rows), threads, 0, stream>>>(
+          KK_ARGS);
+    else
+      embed_streams_kernel<T, 1><<<dim3((unsigned)rows), threads, 0, stream>>>(
+          KK_ARGS);
   });
+#undef KK_ARGS
   HIP_CHECK_KERNEL();
-}
-
-// 4 consecutive elements in the storage format
-DEV_INLINE void ld4(const float* p, float* o) {
-  const float4 a = *reinterpret_cast<const float4*>(p);
-  o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w;
-}
-DEV_INLINE void ld4(const bf16_t* p, float* o) {
-  const uint2 a = *reinterpret_cast<const uint2*>(p);
-  o[0] = us2f((unsigned short)(a.x & 0xffffu)); o[1] = us2f((unsigned short)(a.x >> 16));
-  o[2] = us2f((unsigned short)(a.y & 0xffffu)); o[3] = us2f((unsigned short)(a.y >> 16));
-}
-DEV_INLINE void st4(float* p, const float* v) {
-  *reinterpret_cast<float4*>(p) = float4{v[0], v[1], v[2], v[3]};
-}
-DEV_INLINE void st4(bf16_t* p, const float* v) {
-  *reinterpret_cast<uint2*>(p) =
-      uint2{(unsigned)f2us(v[0]) | ((unsigned)f2us(v[1]) << 16),
-            (unsigned)f2us(v[2]) | ((unsigned)f2us(v[3]) << 16)};
 }
 
 // WRITE: first the streams' update from y, then the read. The blend u waits
