@@ -59,7 +59,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
     int I, int N) {
   constexpr int NP = LN * NR;
   constexpr int NC = 256 / LN;
-  constexpr int TT = PF == 1 ? 1 : SS_TT;
+  constexpr int TT = PF == 1 ? 1 : (NP > 128 ? SS_TT / 2 : SS_TT);
   __shared__ __align__(16) float sB[TT * NP];
   __shared__ __align__(16) float sC[TT * NP];
   const int s = blockIdx.x;
@@ -119,12 +119,13 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
     __syncthreads();
     if (PF == 1 && t0 == 0) {
       if (tid < NP) { sB[tid] = pb; sC[tid] = pc; }
-    } else
-    for (int i = tid; i < nt * NP; i += 256) {
-      const int t = i / NP, nn = i - t * NP;
-      const T* row = bc + (row0 + t0 + t) * ldbc + nn;
-      sB[i] = nn < N ? ldf(row + b_col) : 0.f;
-      sC[i] = nn < N ? ldf(row + c_col) : 0.f;
+    } else {
+      for (int i = tid; i < nt * NP; i += 256) {
+        const int t = i / NP, nn = i - t * NP;
+        const T* row = bc + (row0 + t0 + t) * ldbc + nn;
+        sB[i] = nn < N ? ldf(row + b_col) : 0.f;
+        sC[i] = nn < N ? ldf(row + c_col) : 0.f;
+      }
     }
     __syncthreads();
     for (int t1 = 0; t1 < nt; t1 += PF) {
@@ -225,7 +226,7 @@ void selective_scan(torch::Tensor out, torch::Tensor x, torch::Tensor z,
   const long nseq = cu_rows.numel() - 1;
   TORCH_CHECK(nseq >= 0 && state_slots.numel() >= nseq);
   if (rows == 0 || nseq == 0) return;
-  TORCH_CHECK(N >= 1 && N <= 128, "selective_scan: 1 to 128 states per channel");
+  TORCH_CHECK(N >= 1 && N <= 256, "selective_scan: 1 to 256 states per channel");
   auto stream = c10::hip::getCurrentHIPStream().stream();
 #define KK_LAUNCH(LN_, NR_, PF_)                                                 \
   {                                                                           \
@@ -256,7 +257,8 @@ void selective_scan(torch::Tensor out, torch::Tensor x, torch::Tensor z,
     else if (N <= 16) { KK_PICK(4, 4, 1, 16) }
     else if (N <= 32) { KK_PICK(8, 4, 2, 16) }
     else if (N <= 64) { KK_PICK(16, 4, 4, 16) }
-    else { KK_PICK(16, 8, 8, 16) }
+    else if (N <= 128) { KK_PICK(16, 8, 8, 16) }
+    else { KK_PICK(16, 16, 16, 16) }
   });
 #undef KK_PICK
 #undef KK_LAUNCH

@@ -40,7 +40,8 @@ def test_op_delta(sizes, dtype):
 
 @BOTH
 @pytest.mark.parametrize("sizes", [(9, 5), (24, 1), (300, 8), (64, 16),
-                                   (40, 24), (17, 40), (33, 70), (20, 128)])
+                                   (40, 24), (17, 40), (33, 70), (20, 128),
+                                   (12, 200)])
 def test_op_selective(sizes, dtype):
     cases.case_op_selective(DEV, dtype, *sizes)
     cases.case_op_selective(DEV, dtype, *sizes, cuts=(70, 1, 3, 33, 2))
