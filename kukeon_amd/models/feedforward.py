@@ -1,8 +1,9 @@
 """Feed-forward sublayers beyond the SwiGLU of the Llama family: a dense
 layer with the xIELU activation, a mixture of small experts chosen by a
 per-token-id table (no learned router at run time), a gated dense layer with
-the tanh form of gelu, and a mixture of clamped gated experts chosen by a
-learned router, the weights on their outputs or their inputs."""
+the tanh form of gelu, a dense layer with a squared relu, and a mixture of
+gated experts chosen by a learned router, the weights on their outputs or their
+inputs."""
 from __future__ import annotations
 
 import math
@@ -29,12 +30,15 @@ class FFCfg:
     # "top": weights = softmax over the chosen logits; "all": scores =
     # softmax over all logits, the chosen scores divided by their sum and
     # multiplied by route_scale; "sigmoid": every logit's own sigmoid times
-    # route_scale, not renormalised
+    # route_scale, not renormalised; "corrected": the same scores, chosen by
+    # score plus a learned correction per expert, the chosen scores (without
+    # it) divided by their sum and multiplied by route_scale
     score: str = "top"
     # the weights multiply the experts' inputs instead of their outputs
     weigh_input: bool = False
     groups: int = 0          # experts in this many equal runs of neighbours,
     keep: int = 0            # of which only the best `keep` can be chosen
+    group_best: int = 1      # a run counts the sum of its 1 or 2 best scores
     route_scale: float = 1.0
     shared_ff: int = 0       # hidden size of an always-on expert (0: none)
 
@@ -193,6 +197,29 @@ class GeluGatedFF(nn.Module):
         return ops.linear(a, self.w_down)
 
 
+class SquaredReluFF(nn.Module):
+    """down(max(up h, 0)^2)."""
+
+    def __init__(self, f: FFCfg, width: int, t: Dict[str, torch.Tensor],
+                 p: str, device, dtype):
+        super().__init__()
+        dev = dict(device=device, dtype=dtype)
+        self.w_up = nn.Parameter(t[p + "up"].to(**dev).contiguous(),
+                                 requires_grad=False)
+        self.w_down = nn.Parameter(t[p + "down"].to(**dev).contiguous(),
+                                   requires_grad=False)
+
+    @staticmethod
+    def tensor_shapes(f: FFCfg, width: int, vocab: int) -> Dict[str, tuple]:
+        return {"up": (f.ff, width), "down": (width, f.ff)}
+
+    def forward(self, h: torch.Tensor, ids: torch.Tensor,
+                meta=None) -> torch.Tensor:
+        z = ops.linear(h, self.w_up)
+        ops.relu_square_(z)
+        return ops.linear(z, self.w_down)
+
+
 class RoutedMoE(nn.Module):
     """`experts` small gated feed-forward layers without biases; a token
     uses the `top` experts with the largest router logits, weighted by the
@@ -204,7 +231,8 @@ class RoutedMoE(nn.Module):
     (`act`); scores from a softmax over ALL logits, the chosen ones divided
     by their sum and scaled, the choice limited to the best `keep` of
     `groups` runs of neighbouring experts (`score`, `groups`); scores that
-    are each logit's own sigmoid, used as they are (`score`); weights on the
+    are each logit's own sigmoid, used as they are, or chosen by score plus
+    correction and divided by their sum (`score`); weights on the
     experts' inputs, act(w gate h) * (w up h), where they enter as a factor
     of the two products in fp32 (`weigh_input`); an always-on shared expert
     of the same form (`shared_ff`), added with weight 1. Weights are stacked
@@ -227,11 +255,14 @@ class RoutedMoE(nn.Module):
         if not (0 < f.top <= f.experts):
             raise ValueError(f"{p}: top must be within 1 .. experts")
         if f.act not in ("clamp", "silu") or f.score not in (
-                "top", "all", "sigmoid"):
+                "top", "all", "sigmoid", "corrected"):
             raise ValueError(f"{p}: unknown expert or router kind")
         if f.groups:
-            if f.score != "all" or f.experts % f.groups or \
+            if f.score not in ("all", "corrected") or \
+                    f.experts % f.groups or \
                     not (0 < f.keep <= f.groups) or \
+                    f.group_best not in ((1,) if f.score == "all"
+                                         else (1, 2)) or \
                     f.top > f.keep * (f.experts // f.groups):
                 raise ValueError(f"{p}: expert groups do not fit the router")
         self.f = f
@@ -264,6 +295,10 @@ class RoutedMoE(nn.Module):
         # in the activation format: products of two bf16 numbers are exact
         # in fp32, so the fp32-output GEMM over bf16 rows IS the fp32 router
         self.w_router = t[p + "router"].to(**dev).contiguous()
+        self.correction = None
+        if f.score == "corrected":
+            self.correction = t[p + "correction"].to(
+                device=device, dtype=torch.float32).contiguous()
         if f.score != "top" and f.experts % 16:
             # the score product is made 16 columns wide at least (zero rows
             # below the experts'); the router reads the first `experts`
@@ -272,6 +307,8 @@ class RoutedMoE(nn.Module):
     @staticmethod
     def tensor_shapes(f: FFCfg, width: int, vocab: int) -> Dict[str, tuple]:
         out = {"router": (f.experts, width)}
+        if f.score == "corrected":
+            out["correction"] = (f.experts,)
         for e in range(f.experts):
             out[f"e{e}.gate"] = (f.ff, width)
             out[f"e{e}.up"] = (f.ff, width)
@@ -287,6 +324,10 @@ class RoutedMoE(nn.Module):
         f = self.f
         if f.score == "sigmoid":
             ops.router_sigmoid(idx, wts, logits, f.top, f.route_scale)
+        elif f.score == "corrected":
+            ops.router_corrected(idx, wts, logits, self.correction, f.top,
+                                 f.groups, f.keep, f.group_best,
+                                 f.route_scale, True)
         elif f.score == "all":
             ops.router_select(idx, wts, logits, f.top, f.groups, f.keep,
                               f.route_scale, 0)

@@ -18,6 +18,7 @@ import torch.nn as nn
 
 from kukeon_amd import ops
 from kukeon_amd.engine.kv_cache import LayerKVSpec
+from kukeon_amd.models.rotary import pairs_from_half
 
 
 def _pad8(n: int) -> int:
@@ -175,18 +176,10 @@ class LatentAttnCfg:
     # entry i + rot_dims/2
     rot_layout: str = "pairs"
     # "head": one gate per head (g [H, W]); "element": one per output entry
-    # (g [H*vdim, W])
+    # (g [H*vdim, W]); "none": the heads go to the output projection as is
     gate: str = "head"
-
-
-def _pairs_from_half(dims: int, n: int) -> torch.Tensor:
-    """Row order that turns the half layout of a rotated part of n entries
-    into the pair layout: new[2i] = old[i], new[2i+1] = old[i + dims/2]."""
-    half = dims // 2
-    order = []
-    for i in range(half):
-        order += [i, i + half]
-    return torch.tensor(order + list(range(dims, n)), dtype=torch.long)
+    rot_scaling: tuple = ()  # frequency rescaling (rotary.scaling_key)
+    sink: bool = False       # a learned score per head without a value
 
 
 class LatentAttention(nn.Module):
@@ -201,9 +194,10 @@ class LatentAttention(nn.Module):
 
     so the kernel reads each cache row once for all heads. Queries pass
     their own normed latent (q_rank), or come straight from the input when
-    q_rank is 0. A sliding window may bound the keys, and the output is
-    scaled by sigmoid of a gate projected from the mixer's input, per head
-    or per entry.
+    q_rank is 0. A sliding window may bound the keys, a learned score per
+    head without a value may join the softmax (a sink), and the output may
+    be scaled by sigmoid of a gate projected from the mixer's input, per
+    head or per entry.
 
     The kernels turn pairs (2i, 2i+1). A checkpoint in the half layout
     (entry i with i + rot_dims/2) has the rows of the rotated parts of its
@@ -212,8 +206,8 @@ class LatentAttention(nn.Module):
 
     Tensors (prefix p): dq [q_rank, W], dq.norm, uq [H*(dim+rot_dim), q_rank]
     (or q [H*(dim+rot_dim), W] when q_rank is 0), dkv [kv_rank+rot_dim, W],
-    dkv.norm, uk [H*dim, kv_rank], uv [H*vdim, kv_rank], g [H or H*vdim, W],
-    o [W, H*vdim]."""
+    dkv.norm, uk [H*dim, kv_rank], uv [H*vdim, kv_rank], g [H or H*vdim, W]
+    (with a gate), sink [H] (with a sink), o [W, H*vdim]."""
 
     def __init__(self, m: LatentAttnCfg, width: int, eps: float,
                  t: Dict[str, torch.Tensor], p: str, device, dtype):
@@ -222,7 +216,7 @@ class LatentAttention(nn.Module):
             raise ValueError(f"{p}: bad rotary dims")
         if m.rot_layout not in ("pairs", "half"):
             raise ValueError(f"{p}: unknown rotary layout {m.rot_layout!r}")
-        if m.gate not in ("head", "element"):
+        if m.gate not in ("head", "element", "none"):
             raise ValueError(f"{p}: unknown gate kind {m.gate!r}")
         self.m = m
         self.eps = eps
@@ -231,15 +225,18 @@ class LatentAttention(nn.Module):
         w_q = t[p + ("uq" if m.q_rank else "q")]
         w_dkv = t[p + "dkv"]
         if m.rot_layout == "half":
-            order = _pairs_from_half(m.rot_dims, m.rot_dim)
+            order = pairs_from_half(m.rot_dims, m.rot_dim)
             w_q = w_q.view(H, hd, -1)
             w_q = torch.cat([w_q[:, :m.dim], w_q[:, m.dim:][:, order]],
                             1).reshape(H * hd, -1)
             w_dkv = torch.cat([w_dkv[:R], w_dkv[R:][order]], 0)
         first = ("q", t[p + "dq"] if m.q_rank else w_q)
-        self.col, self.w_down = fuse_rows(
-            [first, ("kv", w_dkv), ("g", t[p + "g"])], width, dtype, device)
+        segs = [first, ("kv", w_dkv)]
+        if m.gate != "none":
+            segs.append(("g", t[p + "g"]))
+        self.col, self.w_down = fuse_rows(segs, width, dtype, device)
         f32 = dict(device=device, dtype=torch.float32)
+        self.sinks = t[p + "sink"].to(**f32).contiguous() if m.sink else None
         self.q_norm = (t[p + "dq.norm"].to(**f32).contiguous() if m.q_rank
                        else torch.empty(0, **f32))
         self.kv_norm = t[p + "dkv.norm"].to(**f32).contiguous()
@@ -248,7 +245,8 @@ class LatentAttention(nn.Module):
         if m.q_rank:
             self.w_uq = nn.Parameter(w_q.to(**dev).contiguous(),
                                      requires_grad=False)
-        self.gate_cols = H if m.gate == "head" else H * m.vdim
+        self.gate_cols = {"head": H, "element": H * m.vdim,
+                          "none": 0}[m.gate]
         # [H, dim, R]: q_abs_h = q_h W_uk_h;  [H, R, vdim]: o_h = l_h W_uv_h^T
         self.w_uk = nn.Parameter(t[p + "uk"].to(**dev).view(H, m.dim, R)
                                  .contiguous(), requires_grad=False)
@@ -265,8 +263,11 @@ class LatentAttention(nn.Module):
         out = {"dkv": (m.kv_rank + m.rot_dim, width),
                "dkv.norm": (m.kv_rank,), "uk": (H * m.dim, m.kv_rank),
                "uv": (H * m.vdim, m.kv_rank),
-               "g": (H if m.gate == "head" else H * m.vdim, width),
                "o": (width, H * m.vdim)}
+        if m.gate != "none":
+            out["g"] = (H if m.gate == "head" else H * m.vdim, width)
+        if m.sink:
+            out["sink"] = (H,)
         if m.q_rank:
             out.update({"dq": (m.q_rank, width), "dq.norm": (m.q_rank,),
                         "uq": (H * (m.dim + m.rot_dim), m.q_rank)})
@@ -300,11 +301,13 @@ class LatentAttention(nn.Module):
         lat = torch.empty(H, T, R, dtype=h.dtype, device=h.device)
         ops.latent_attention(lat, q_abs, q, cache, self.cs, meta.positions,
                              meta.row_seq, meta.block_table, H, m.dim,
-                             m.rot_dim, m.window, m.scale)
+                             m.rot_dim, m.window, m.scale, self.sinks)
         o = torch.bmm(lat, self.w_uv)                  # [H, T, vdim]
         og = torch.empty(T, H * m.vdim, dtype=h.dtype, device=h.device)
-        ops.head_gate(og, o, proj[:, self.col["g"]:
-                                  self.col["g"] + self.gate_cols])
+        gate = None
+        if self.gate_cols:
+            gate = proj[:, self.col["g"]: self.col["g"] + self.gate_cols]
+        ops.head_gate(og, o, gate)
         return ops.linear(og, self.w_o)
 
 
@@ -997,6 +1000,8 @@ class SinkAttention(nn.Module):
         if m.log_bias:
             self.r1 = t[p + "r1"].to(**f32).contiguous()
             self.r2 = t[p + "r2"].to(**f32).contiguous()
+        # the 1 in the denominator is a score of 0
+        self.sinks = torch.zeros(m.heads, **f32) if m.sink else None
         self.w_o = nn.Parameter(t[p + "o"].to(device=device, dtype=dtype)
                                 .contiguous(), requires_grad=False)
 
@@ -1030,16 +1035,16 @@ class SinkAttention(nn.Module):
                 meta.qb_seq is not None and
                 ops.masked_tiles_supported(q, m.dim, cache.shape[2])):
             # prompt portions on the matrix cores
-            ops.masked_attention_tiles(o, q, cache, self.r1, self.r2,
-                                       meta.block_table, meta.seq_lens,
-                                       meta.q_starts, meta.qb_seq,
-                                       meta.qb_start, m.scale, m.softcap,
-                                       m.chunk, m.sink, self.eps)
+            ops.masked_attention_tiles(o, q, cache, None, self.r1, self.r2,
+                                       self.sinks, meta.block_table,
+                                       meta.seq_lens, meta.q_starts,
+                                       meta.qb_seq, meta.qb_start, m.scale,
+                                       m.softcap, m.chunk, 0, self.eps)
         else:
             ops.masked_attention(o, q, cache, None, None, self.r1, self.r2,
                                  meta.positions, meta.row_seq,
                                  meta.block_table, m.heads, m.scale,
-                                 m.softcap, m.chunk, 0, m.sink, self.eps)
+                                 m.softcap, m.chunk, 0, self.sinks, self.eps)
         og = torch.empty_like(o)
         ops.scaled_gate(og, o, proj[:, c["g"]: c["g"] + self.Cq], 1)
         return ops.linear(og, self.w_o)
@@ -1153,3 +1158,102 @@ class SelectiveMixer(nn.Module):
                            self.dt_bias, dbc, c["B"], c["C"], self.A2, self.D,
                            S, meta.positions, meta.cu_rows, meta.state_slots)
         return ops.linear(y, self.w_o)
+
+
+# ---------------------------------------------------------------------------
+@dataclass
+class RotaryAttnCfg:
+    heads: int
+    kv_heads: int
+    dim: int                 # query/key entries per head
+    vdim: int                # value entries per head
+    scale: float
+    rot_dims: int = 0        # leading entries of a head that turn (0: none)
+    rot_base: float = 10000.0
+    rot_scaling: tuple = ()  # frequency rescaling (rotary.scaling_key)
+    # "half": entry i turns with entry i + rot_dims/2; "pairs": (2i, 2i+1)
+    rot_layout: str = "half"
+    window: int = 0          # position i sees i-window+1 .. i (0: all)
+    keep_first: int = 0      # and, with a window, the first positions
+    sink: bool = False       # a learned score per head without a value
+
+
+class RotaryAttention(nn.Module):
+    """Grouped-query softmax attention with rotary positions on the first
+    `rot_dims` entries of every query and key head. A sliding window may
+    bound the keys; position i then sees j <= i with i - j < window or
+    j < keep_first, the kept ones at their own positions. With a sink the
+    softmax has one more learned score per head that has no key and no value.
+
+    The kernels turn pairs (2i, 2i+1); a checkpoint in the half layout has
+    the rows of its query and key projections reordered at load (a score is
+    a dot product over those rows, so only its order of summation changes).
+
+    Tensors (prefix p): q [H*dim, W], k [G*dim, W], v [G*vdim, W], sink [H]
+    (with a sink), o [W, H*vdim]."""
+
+    def __init__(self, m: RotaryAttnCfg, width: int, eps: float,
+                 t: Dict[str, torch.Tensor], p: str, device, dtype):
+        super().__init__()
+        if m.heads % m.kv_heads:
+            raise ValueError(f"{p}: heads not a multiple of kv_heads")
+        if m.rot_dims % 2 or m.rot_dims > m.dim:
+            raise ValueError(f"{p}: bad rotary dims")
+        if m.rot_layout not in ("pairs", "half"):
+            raise ValueError(f"{p}: unknown rotary layout {m.rot_layout!r}")
+        self.m = m
+        w_q, w_k = t[p + "q"], t[p + "k"]
+        if m.rot_layout == "half":
+            order = pairs_from_half(m.rot_dims, m.dim).to(w_q.device)
+            w_q, w_k = (w.view(-1, m.dim, width)[:, order].reshape(-1, width)
+                        for w in (w_q, w_k))
+        self.col, self.w_in = fuse_rows(
+            [("q", w_q), ("k", w_k), ("v", t[p + "v"])], width, dtype, device)
+        f32 = dict(device=device, dtype=torch.float32)
+        self.sinks = t[p + "sink"].to(**f32).contiguous() if m.sink else None
+        self.w_o = nn.Parameter(t[p + "o"].to(device=device, dtype=dtype)
+                                .contiguous(), requires_grad=False)
+        self.cs = None       # angle table [positions, rot_dims], set by the model
+
+    @staticmethod
+    def tensor_shapes(m: RotaryAttnCfg, width: int) -> Dict[str, tuple]:
+        out = {"q": (m.heads * m.dim, width), "k": (m.kv_heads * m.dim, width),
+               "v": (m.kv_heads * m.vdim, width),
+               "o": (width, m.heads * m.vdim)}
+        if m.sink:
+            out["sink"] = (m.heads,)
+        return out
+
+    def kv_spec(self) -> Optional[LayerKVSpec]:
+        return LayerKVSpec(self.m.kv_heads, self.m.dim, self.m.vdim)
+
+    def state_shape(self):
+        return None
+
+    def forward(self, h: torch.Tensor, cache, state, meta,
+                cache_v=None) -> torch.Tensor:
+        m = self.m
+        T = h.shape[0]
+        c = self.col
+        proj = ops.linear(h, self.w_in)
+        q = torch.empty(T, m.heads * m.dim, dtype=h.dtype, device=h.device)
+        ops.rotary_append(q, cache, cache_v, proj, c["q"], c["k"], c["v"],
+                          self.cs, meta.positions, meta.row_seq,
+                          meta.block_table)
+        o = torch.empty(T, m.heads * m.vdim, dtype=h.dtype, device=h.device)
+        if (meta.mode == "prefill" and meta.max_rows >= 16 and
+                meta.qb_seq is not None and
+                ops.masked_tiles_supported(q, m.dim, cache.shape[2], m.vdim)):
+            # prompt portions on the matrix cores
+            ops.masked_attention_tiles(o, q, cache, cache_v, None, None,
+                                       self.sinks, meta.block_table,
+                                       meta.seq_lens, meta.q_starts,
+                                       meta.qb_seq, meta.qb_start, m.scale,
+                                       window=m.window, keep=m.keep_first)
+        else:
+            ops.masked_attention(o, q, cache, cache_v, None, None, None,
+                                 meta.positions, meta.row_seq,
+                                 meta.block_table, m.heads, m.scale,
+                                 window=m.window, sinks=self.sinks,
+                                 keep=m.keep_first)
+        return ops.linear(o, self.w_o)

@@ -47,6 +47,11 @@ def _noridra(cfg, device, **kw):
     return NoridraModel(cfg, device=device, **kw)
 
 
+def _senavik(cfg, device, **kw):
+    from kukeon_amd.models.senavik import SenavikModel
+    return SenavikModel(cfg, device=device, **kw)
+
+
 # family -> constructor(cfg, device, **kw)
 FAMILIES: Dict[str, Callable] = {
     "bezizen": _bezizen,
@@ -56,6 +61,7 @@ FAMILIES: Dict[str, Callable] = {
     "lipedra": _lipedra,
     "noridra": _noridra,
     "rasesun": _rasesun,
+    "senavik": _senavik,
 }
 
 # config.json "architecture" -> family
@@ -65,6 +71,7 @@ ARCHITECTURES: Dict[str, str] = {
     "Dumovik": "dumovik",
     "Bezizen": "bezizen",
     "Noridra": "noridra",
+    "Senavik": "senavik",
 }
 
 
@@ -78,6 +85,7 @@ OP_GROUPS: Dict[str, tuple] = {
     "dumovik": ("hyb",),
     "bezizen": ("strm",),
     "noridra": ("delta",),
+    "senavik": ("sink",),
 }
 
 
@@ -190,27 +198,38 @@ NORIDRA_PRESETS = {
 }
 
 
+def _senavik_preset(**kw):
+    def make():
+        from kukeon_amd.models.senavik import senavik_bench
+        return senavik_bench(**kw)
+    return make
+
+
+# random-weight Senavik stacks: three windowed attention layers to one latent
+# attention layer at Llama-3-8B width, and a small one
+SENAVIK_PRESETS = {
+    "senavik-8b-like": _senavik_preset(width=4096, layers=32, heads=32,
+                                       kv_heads=8, ff=14336, vocab=128256,
+                                       name="senavik-8b-like"),
+    "tiny-senavik": _senavik_preset(width=128, layers=4, heads=4, kv_heads=2,
+                                    ff=256, vocab=384, window=24, experts=8,
+                                    name="tiny-senavik"),
+}
+
+_PRESETS = (MODEL_PRESETS, LIPEDRA_PRESETS, RASESUN_PRESETS, DUMOVIK_PRESETS,
+            BEZIZEN_PRESETS, NORIDRA_PRESETS, SENAVIK_PRESETS)
+
+
 def preset_names():
-    return sorted(list(MODEL_PRESETS) + list(LIPEDRA_PRESETS) +
-                  list(RASESUN_PRESETS) + list(DUMOVIK_PRESETS) +
-                  list(BEZIZEN_PRESETS) + list(NORIDRA_PRESETS))
+    return sorted(name for group in _PRESETS for name in group)
 
 
 def preset(name: str):
-    if name in NORIDRA_PRESETS:
-        return NORIDRA_PRESETS[name]()
-    if name in BEZIZEN_PRESETS:
-        return BEZIZEN_PRESETS[name]()
-    if name in DUMOVIK_PRESETS:
-        return DUMOVIK_PRESETS[name]()
-    if name in LIPEDRA_PRESETS:
-        return LIPEDRA_PRESETS[name]()
-    if name in RASESUN_PRESETS:
-        return RASESUN_PRESETS[name]()
-    if name not in MODEL_PRESETS:
-        raise KeyError(f"unknown model preset {name!r}; known: "
-                       f"{preset_names()}")
-    return MODEL_PRESETS[name]()
+    for group in _PRESETS:
+        if name in group:
+            return group[name]()
+    raise KeyError(f"unknown model preset {name!r}; known: "
+                   f"{preset_names()}")
 
 
 def load_checkpoint(model_dir: str, device, dtype: str = "bf16"):
@@ -240,5 +259,9 @@ def load_checkpoint(model_dir: str, device, dtype: str = "bf16"):
     if fam == "noridra":
         from kukeon_amd.models.noridra import NoridraModel
         return NoridraModel.from_checkpoint(model_dir, device=device,
+                                            dtype=dtype)
+    if fam == "senavik":
+        from kukeon_amd.models.senavik import SenavikModel
+        return SenavikModel.from_checkpoint(model_dir, device=device,
                                             dtype=dtype)
     raise ValueError(f"family {fam} has no checkpoint loader")

@@ -193,6 +193,42 @@ def _delta(t: torch.Tensor):
     return _C_delta
 
 
+_C_sink = None
+_SINK_IMPORT_ERROR: Exception | None = None
+try:
+    from kukeon_amd import _C_sink  # type: ignore
+except Exception as e:  # pragma: no cover
+    _SINK_IMPORT_ERROR = e
+
+
+def sink_available() -> bool:
+    return _C_sink is not None
+
+
+def _sink(t: torch.Tensor):
+    """Kernel group of the stacks whose softmax has a sink per head (normed
+    embedding rows, partial rotary positions, windowed attention with kept
+    first tokens, latent attention, corrected sigmoid routing): native on a
+    GPU tensor (an error if the module is not built), fp32 references on
+    CPU."""
+    global _C_sink, _SINK_IMPORT_ERROR
+    if not t.is_cuda:
+        return reference
+    if _C_sink is None:
+        try:
+            import importlib
+            _C_sink = importlib.import_module("kukeon_amd._C_sink")
+        except Exception as e:
+            _SINK_IMPORT_ERROR = e
+    if _C_sink is None:
+        raise RuntimeError(
+            "kukeon_amd._C_sink (gfx950 HIP extension) is not built but an "
+            "op was called on a CUDA device. Run `python -m "
+            f"kukeon_amd.ops.build sink` (import error: "
+            f"{_SINK_IMPORT_ERROR})")
+    return _C_sink
+
+
 _SHARED_CHOICE: dict = {}
 
 
@@ -503,7 +539,7 @@ def residual_add_rmsnorm(x, a, bias, w, w_offset: float, eps: float,
                          out) -> None:
     """x (fp32 residual, in place) += a (+ bias); out = rmsnorm(x) scaled by
     (w_offset + w). `a` / `bias` may be None."""
-    _mix(x).residual_add_rmsnorm(
+    _shared(x, _mix, _sink).residual_add_rmsnorm(
         x, a if a is not None else _e(out),
         bias if bias is not None else _e(x), w, w_offset, eps, out)
 
@@ -513,7 +549,7 @@ def clamp_glu(out, gate, up, bg, bu, limit: float, alpha: float = 1.702,
     """`row_scale` [T] multiplies a row's gate and up ahead of everything
     else."""
     none = torch.empty(0, dtype=torch.float32, device=out.device)
-    _shared(out, _mix, _hyb, _strm, _delta).clamp_glu(
+    _shared(out, _mix, _hyb, _strm, _delta, _sink).clamp_glu(
         out, gate, up, bg if bg is not None else none,
         bu if bu is not None else none, limit, alpha, up_shift,
         row_scale if row_scale is not None else none)
@@ -649,21 +685,27 @@ def gated_group_rmsnorm(out, y, z, w, groups: int, eps: float) -> None:
 def latent_kv_append(cq_out, cache, proj, q_col: int, kv_col: int, wq, wkv,
                      eps: float, cs, positions, row_seq,
                      block_table) -> None:
-    _shared(proj, _recur, _hyb).latent_kv_append(
+    _shared(proj, _recur, _hyb, _sink).latent_kv_append(
         cq_out, cache, proj, q_col, kv_col, wq, wkv, eps, cs, positions,
         row_seq, block_table)
 
 
 def latent_attention(out, q_abs, q, cache, cs, positions, row_seq,
                      block_table, H: int, dn: int, dr: int, window: int,
-                     scale: float) -> None:
-    _shared(q, _recur, _hyb).latent_attention(
+                     scale: float, sinks=None) -> None:
+    """`sinks` [H]: one more score per head in the softmax, without a
+    latent."""
+    _shared(q, _recur, _hyb, _sink).latent_attention(
         out, q_abs, q, cache, cs, positions, row_seq, block_table, H, dn, dr,
-        window, scale)
+        window, scale, sinks if sinks is not None
+        else torch.empty(0, dtype=torch.float32, device=q.device))
 
 
 def head_gate(out, o, gate) -> None:
-    _shared(out, _recur, _hyb).head_gate(out, o, gate)
+    """o [H, T, dv] -> out [T, H*dv], times sigmoid of `gate` unless that is
+    None."""
+    _shared(out, _recur, _hyb, _sink).head_gate(
+        out, o, gate if gate is not None else _e(out))
 
 
 def xielu(out, z, ap: float, aq: float) -> None:
@@ -675,11 +717,12 @@ def table_moe(out, h, ids, table, w_up, w_down) -> None:
 
 
 def gather_rows(out, inp, row_map) -> None:
-    _shared(out, _recur, _hyb, _strm, _delta).gather_rows(out, inp, row_map)
+    _shared(out, _recur, _hyb, _strm, _delta, _sink).gather_rows(out, inp,
+                                                                 row_map)
 
 
 def relu_square_(x) -> None:
-    _recur(x).relu_square_(x)
+    _shared(x, _recur, _sink).relu_square_(x)
 
 
 def combine_rows(out, inp, inv) -> None:
@@ -759,7 +802,8 @@ def router_topk(idx, wts, logits, top: int, dense_rows: int = 0) -> None:
 
 
 def combine_rows_weighted(out, inp, inv, wts) -> None:
-    _shared(out, _hyb, _strm, _delta).combine_rows_weighted(out, inp, inv, wts)
+    _shared(out, _hyb, _strm, _delta, _sink).combine_rows_weighted(
+        out, inp, inv, wts)
 
 
 # ---- stream group ----------------------------------------------------------
@@ -875,7 +919,7 @@ def routed_experts(out, h, idx, wts, top: int, w_gu, w_down, limit: float,
     """The chosen experts of a small batch: idx, wts [T, >= top]; the
     weights multiply the experts' outputs, or their inputs; `extra` [T, W]
     is added last."""
-    _shared(h, _hyb, _strm, _delta).routed_experts(
+    _shared(h, _hyb, _strm, _delta, _sink).routed_experts(
         out, h, idx, wts, top, w_gu, w_down, limit, alpha, shift, weigh_input,
         extra if extra is not None else _e(h))
 
@@ -938,37 +982,75 @@ def head_norm_append(q_out, k_cache, proj, q_col: int, k_col: int, w,
 def masked_attention(out, q, k_cache, v_cache, slopes, r1, r2, positions,
                      row_seq, block_table, H: int, scale: float,
                      softcap: float = 0.0, chunk: int = 0, window: int = 0,
-                     sink: bool = False, key_eps: float = -1.0) -> None:
+                     sinks=None, key_eps: float = -1.0,
+                     keep: int = 0) -> None:
     """Softmax attention over paged keys with every option of the row kernel:
     values are the keys when v_cache is None; a linear (slopes) and a
     logarithmic (r1, r2) distance bias, capped scores, chunk and window,
-    a sink of score 0, keys divided by their root mean square (key_eps >=
+    the first `keep` positions visible besides, a score without a value per
+    head (sinks [H]), keys divided by their root mean square (key_eps >=
     0)."""
     none = torch.empty(0, dtype=torch.float32, device=q.device)
     o = lambda t: t if t is not None else none
-    _delta(q).masked_attention(
+    _shared(q, _delta, _sink).masked_attention(
         out, q, k_cache, v_cache if v_cache is not None else _e(q), o(slopes),
-        o(r1), o(r2), positions, row_seq, block_table, H, scale, softcap,
-        chunk, window, sink, key_eps)
+        o(r1), o(r2), o(sinks), positions, row_seq, block_table, H, scale,
+        softcap, chunk, window, keep, key_eps)
 
 
-def masked_tiles_supported(t: torch.Tensor, d: int, BS: int) -> bool:
+def masked_tiles_supported(t: torch.Tensor, d: int, BS: int,
+                           dv: int = None) -> bool:
+    """Whether the matrix-core kernel for prompt portions serves these
+    sizes (bf16 on a GPU only); `dv` is the value size where the values are
+    not the keys."""
     return (t.is_cuda and t.dtype == torch.bfloat16
-            and _delta(t).masked_attention_tiles_supported(d, BS))
+            and _shared(t, _delta, _sink).chunk_attention_tiles_supported(
+                d, d if dv is None else dv, BS))
 
 
-def masked_attention_tiles(out, q, k_cache, r1, r2, block_table, seq_lens,
-                           q_starts, qb_seq, qb_start, scale: float,
-                           softcap: float, chunk: int, sink: bool,
-                           key_eps: float) -> None:
+def masked_attention_tiles(out, q, k_cache, v_cache, r1, r2, sinks,
+                           block_table, seq_lens, q_starts, qb_seq, qb_start,
+                           scale: float, softcap: float = 0.0,
+                           chunk: int = 0, window: int = 0,
+                           key_eps: float = -1.0, keep: int = 0) -> None:
     none = torch.empty(0, dtype=torch.float32, device=q.device)
-    _delta(q).masked_attention_tiles(
-        out, q, k_cache, r1 if r1 is not None else none,
-        r2 if r2 is not None else none, block_table, seq_lens, q_starts,
-        qb_seq, qb_start, scale, softcap, chunk, sink, key_eps)
+    o = lambda t: t if t is not None else none
+    _shared(q, _delta, _sink).masked_attention_tiles(
+        out, q, k_cache, v_cache if v_cache is not None else _e(q), o(r1),
+        o(r2), o(sinks), block_table, seq_lens, q_starts, qb_seq, qb_start,
+        scale, softcap, chunk, window, keep, key_eps)
 
 
 def router_sigmoid(idx, wts, logits, top: int, scale: float = 1.0) -> None:
     """The `top` experts with the largest logits, weights sigmoid(logit)
     times scale."""
     _delta(logits).router_sigmoid(idx, wts, logits, top, scale)
+
+
+# ---- sink group ------------------------------------------------------------
+def embed_rmsnorm(x, out, ids, table, w, w2, w_offset: float,
+                  eps: float) -> None:
+    """x (fp32) = rmsnorm(table[id]) * (w_offset + w), then
+    out = rmsnorm(x) * (w_offset + w2)."""
+    _sink(x).embed_rmsnorm(x, out, ids, table, w, w2, w_offset, eps)
+
+
+def rotary_append(q_out, k_cache, v_cache, proj, q_col: int, k_col: int,
+                  v_col: int, cs, positions, row_seq, block_table) -> None:
+    """Rotate the first cs.shape[1] entries of every query and key head as
+    pairs (2i, 2i+1); queries to q_out, key and value rows to their page."""
+    _sink(proj).rotary_append(q_out, k_cache, v_cache, proj, q_col, k_col,
+                              v_col, cs, positions, row_seq, block_table)
+
+
+def router_corrected(idx, wts, logits, correction, top: int, groups: int = 0,
+                     keep: int = 0, best: int = 1, scale: float = 1.0,
+                     renorm: bool = False) -> None:
+    """Sigmoid scores; the `top` experts with the largest score plus
+    correction among the `keep` best of `groups` runs of neighbours (a run
+    counts the sum of its `best` largest); weights = the scores without the
+    correction, divided by their sum if `renorm`, times scale."""
+    _sink(logits).router_corrected(
+        idx, wts, logits, correction if correction is not None
+        else torch.empty(0, dtype=torch.float32, device=logits.device), top,
+        groups, keep, best, scale, renorm)

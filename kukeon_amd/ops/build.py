@@ -103,6 +103,24 @@ DELTA_SOURCES = [
     "bindings_delta.cpp",
 ]
 
+#   sink -> kukeon_amd/_C_sink.so  (normed embedding rows, partial rotary
+#                                  positions, windowed attention with kept
+#                                  first tokens and latent attention, both
+#                                  with sinks, corrected sigmoid routing)
+SINK_SOURCES = [
+    "resid_norm.hip",
+    "rotary_append.hip",
+    "chunk_attn.hip",
+    "prefill_attn.hip",
+    "latent_attn.hip",
+    "recur_elem.hip",
+    "routed_moe.hip",
+    "routed_experts.hip",
+    "glu_clamp.hip",
+    "table_moe.hip",
+    "bindings_sink.cpp",
+]
+
 SOURCES = [
     "rmsnorm.hip",
     "activation.hip",
@@ -137,6 +155,7 @@ GROUPS = {
     "hyb": ("_C_hyb", HYB_SOURCES),
     "strm": ("_C_strm", STRM_SOURCES),
     "delta": ("_C_delta", DELTA_SOURCES),
+    "sink": ("_C_sink", SINK_SOURCES),
 }
 
 

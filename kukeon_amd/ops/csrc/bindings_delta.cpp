@@ -45,18 +45,19 @@ void head_norm_append(torch::Tensor q_out, torch::Tensor k_cache,
                       torch::Tensor row_seq, torch::Tensor block_table);
 void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                       torch::Tensor v_cache, torch::Tensor slopes,
-                      torch::Tensor r1, torch::Tensor r2,
+                      torch::Tensor r1, torch::Tensor r2, torch::Tensor sinks,
                       torch::Tensor positions, torch::Tensor row_seq,
                       torch::Tensor block_table, int64_t H, double scale,
                       double softcap, int64_t chunk, int64_t window,
-                      bool sink, double key_eps);
+                      int64_t keep, double key_eps);
 void masked_attention_tiles(torch::Tensor out, torch::Tensor q,
-                            torch::Tensor k_cache, torch::Tensor r1,
-                            torch::Tensor r2, torch::Tensor block_table,
+                            torch::Tensor k_cache, torch::Tensor v_cache,
+                            torch::Tensor r1, torch::Tensor r2,
+                            torch::Tensor sinks, torch::Tensor block_table,
                             torch::Tensor seq_lens, torch::Tensor q_starts,
                             torch::Tensor qb_seq, torch::Tensor qb_start,
                             double scale, double softcap, int64_t chunk,
-                            bool sink, double key_eps);
+                            int64_t window, int64_t keep, double key_eps);
 void scaled_gate(torch::Tensor out, torch::Tensor a, torch::Tensor gate,
                  int64_t act, double scale);
 void router_sigmoid(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
@@ -71,7 +72,7 @@ void clamp_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
                torch::Tensor bg, torch::Tensor bu, double limit, double alpha,
                double up_shift, torch::Tensor row_scale);
 void gather_rows(torch::Tensor out, torch::Tensor in, torch::Tensor map);
-bool window_attention_tiles_supported(int64_t d, int64_t BS);
+bool chunk_attention_tiles_supported(int64_t d, int64_t dv, int64_t BS);
 }  // namespace kukeon
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -107,6 +108,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "clamped gate * sigmoid(alpha gate) * (up + shift)");
   m.def("gather_rows", &kukeon::gather_rows,
         "out[r] = in[map[r]]");
-  m.def("masked_attention_tiles_supported",
-        &kukeon::window_attention_tiles_supported);
+  m.def("chunk_attention_tiles_supported",
+        &kukeon::chunk_attention_tiles_supported);
 }

@@ -57,7 +57,8 @@ void latent_attention(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q,
                       torch::Tensor cache, torch::Tensor cs,
                       torch::Tensor positions, torch::Tensor row_seq,
                       torch::Tensor block_table, int64_t H, int64_t dn,
-                      int64_t dr, int64_t window, double scale);
+                      int64_t dr, int64_t window, double scale,
+                      torch::Tensor sinks);
 void gather_rows(torch::Tensor out, torch::Tensor in, torch::Tensor map);
 }  // namespace kukeon
 

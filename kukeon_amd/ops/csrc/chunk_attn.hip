@@ -7,14 +7,15 @@
 // where the values are the keys (window_attention); and, through
 // masked_attention, a logarithmic distance bias r1_h ln(1 + r2_h (p - j)), keys
 // that are divided by their own root mean square as they are read (the page
-// row stays the value), and a sink, a score of 0 without a value that joins
-// the softmax.
+// row stays the value), a sink per head, a score without a value that joins the
+// softmax, and first tokens that a window keeps.
 //
 // qk_norm_append   norms q (and k) of every row, writes q to a dense buffer
 //                  and k, v to the row's page.
 // chunk_attention  one workgroup per (row, kv head, four of its query heads).
-//                  Keys are taken 64 at a time counted from lo, tile t by
-//                  wave t mod NW: lane j scores key j for all the heads from
+//                  The visible keys (the kept first tokens, then lo .. p) are
+//                  numbered from 0 and taken 64 at a time, tile t by wave
+//                  t mod NW: lane j scores key j for all the heads from
 //                  one read of the key row (the queries sit in LDS as fp32),
 //                  the wave agrees on each head's running maximum and sum,
 //                  then dv/8 lanes cover one value row with 16-byte loads
@@ -209,14 +210,15 @@ struct AttnExtra {
   const float* slopes;     // [H] linear distance bias
   const float* r1;         // [H] logarithmic distance bias
   const float* r2;
+  const float* sinks;      // [H] scores without a value
   float key_eps;           // >= 0: keys divided by their root mean square
-  int sink;
+  int keep;                // first tokens that every query sees
 };
 
 // One workgroup per (row, kv head, up to CA_HB of its query heads). Its NW
 // waves (4 for many rows, 16 for few, where the keys are the only source of
-// parallel work) share out the row's key tiles (tile t of 64 keys, counted
-// from lo, goes to wave t mod NW); every wave serves all the heads from one
+// parallel work) share out the row's key tiles (tile t of 64 visible keys
+// goes to wave t mod NW); every wave serves all the heads from one
 // read of a key or value row. VEC: d and dv multiples of 8 and 16-byte aligned rows;
 // otherwise scalar loads, and lane e owns value entries e, e + 64, ...
 template <typename T, bool VEC>
@@ -286,13 +288,18 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
   const int sub = VEC ? lane - grp * NL : lane;
   const bool vlive = VEC ? grp < NG : true;
 
-  for (int j0 = lo + wave * WAVE; j0 <= p; j0 += NW * WAVE) {
-    const int j = j0 + lane;
+  // visible key n is position n below nkeep, lo + n - nkeep from there on
+  const int nkeep = min(ex.keep, lo);
+  const int nvis = nkeep + p - lo + 1;
+  for (int n0 = wave * WAVE; n0 < nvis; n0 += NW * WAVE) {
+    const int n = n0 + lane;
+    const bool seen = n < nvis;
+    const int j = n < nkeep ? n : lo + n - nkeep;
     float sc[CA_HB];
 #pragma unroll
     for (int hb = 0; hb < CA_HB; ++hb) sc[hb] = -INFINITY;
     long voff = 0;
-    if (j <= p) {
+    if (seen) {
       const long blk = block_table[(long)s * max_blocks + j / BS];
       const long slot = (blk * G + g) * BS + j % BS;
       const T* kr = kc + slot * d;
@@ -338,7 +345,7 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
 #pragma unroll
     for (int hb = 0; hb < CA_HB; ++hb) {
       const float mn = fmaxf(m[hb], wave_max(sc[hb]));
-      const float w = j <= p ? expf(sc[hb] - mn) : 0.f;
+      const float w = seen ? expf(sc[hb] - mn) : 0.f;
       const float alpha = expf(m[hb] - mn);   // m = -inf at first: alpha = 0
       l[hb] = l[hb] * alpha + wave_sum(w);
       m[hb] = mn;
@@ -349,7 +356,7 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
     soff[lane] = voff;
     // wave-private LDS: a wave's LDS operations complete in order
     __builtin_amdgcn_wave_barrier();
-    const int nk = min(WAVE, p - j0 + 1);
+    const int nk = min(WAVE, nvis - n0);
     if (VEC) {
       if (vlive) {
         for (int k = grp; k < nk; k += NG) {
@@ -421,10 +428,11 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
   // fold the waves in wave order; a wave without keys has max -inf, weight 0
   for (int i = tid; i < nh * dv; i += blockDim.x) {
     const int hb = i / dv, e = i - hb * dv;
-    float M = ex.sink ? 0.f : -INFINITY;
+    const float sink = ex.sinks ? ex.sinks[h0 + hb] : -INFINITY;
+    float M = sink;
     for (int w = 0; w < NW; ++w)
       M = fmaxf(M, sml[(w * CA_HB + hb) * 2]);
-    float num = 0.f, den = ex.sink ? expf(-M) : 0.f;
+    float num = 0.f, den = expf(sink - M);
     for (int w = 0; w < NW; ++w) {
       const float f = expf(sml[(w * CA_HB + hb) * 2] - M);
       num = fmaf(f, smo[(w * CA_HB + hb) * dv + e], num);
@@ -435,15 +443,15 @@ __global__ __launch_bounds__(1024) void chunk_attention_kernel(
 }
 
 // out [T, H*dv], q [T, H*d] contiguous; caches as in qk_norm_append. An
-// empty v_cache means that the values are the keys; slopes, r1, r2 [H] fp32 or
-// empty.
+// empty v_cache means that the values are the keys; slopes, r1, r2, sinks [H]
+// fp32 or empty. With a window, positions below `keep` stay visible.
 void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                       torch::Tensor v_cache, torch::Tensor slopes,
-                      torch::Tensor r1, torch::Tensor r2,
+                      torch::Tensor r1, torch::Tensor r2, torch::Tensor sinks,
                       torch::Tensor positions, torch::Tensor row_seq,
                       torch::Tensor block_table, int64_t H, double scale,
                       double softcap, int64_t chunk, int64_t window,
-                      bool sink, double key_eps) {
+                      int64_t keep, double key_eps) {
   check_act(q, "q");
   if (v_cache.numel() == 0) v_cache = k_cache;
   const bool biased = slopes.numel() > 0;
@@ -456,11 +464,17 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
     check_f32(r1, "r1"); check_f32(r2, "r2");
     TORCH_CHECK(r1.numel() == H && r2.numel() == H);
   }
+  const bool sunk = sinks.numel() > 0;
+  if (sunk) {
+    check_f32(sinks, "sinks");
+    TORCH_CHECK(sinks.numel() == H);
+  }
   const AttnExtra ex{biased ? slopes.data_ptr<float>() : nullptr,
                      logb ? r1.data_ptr<float>() : nullptr,
-                     logb ? r2.data_ptr<float>() : nullptr, (float)key_eps,
-                     (int)sink};
-  TORCH_CHECK(window >= 0);
+                     logb ? r2.data_ptr<float>() : nullptr,
+                     sunk ? sinks.data_ptr<float>() : nullptr, (float)key_eps,
+                     (int)keep};
+  TORCH_CHECK(window >= 0 && keep >= 0);
   check_i32(positions, "positions"); check_i32(row_seq, "row_seq");
   check_i32(block_table, "block_table");
   TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous() &&
@@ -542,9 +556,9 @@ void chunk_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                      int64_t H, double scale, double softcap, int64_t chunk) {
   const auto none =
       torch::empty({0}, positions.options().dtype(torch::kFloat32));
-  masked_attention(out, q, k_cache, v_cache, none, none, none, positions,
-                   row_seq, block_table, H, scale, softcap, chunk, 0, false,
-                   -1.0);
+  masked_attention(out, q, k_cache, v_cache, none, none, none, none,
+                   positions, row_seq, block_table, H, scale, softcap, chunk, 0,
+                   0, -1.0);
 }
 
 // Sliding-window attention with a distance bias; an empty v_cache makes the
@@ -556,8 +570,8 @@ void window_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                       int64_t window) {
   const auto none =
       torch::empty({0}, positions.options().dtype(torch::kFloat32));
-  masked_attention(out, q, k_cache, v_cache, slopes, none, none, positions,
-                   row_seq, block_table, H, scale, 0.0, 0, window, false,
+  masked_attention(out, q, k_cache, v_cache, slopes, none, none, none,
+                   positions, row_seq, block_table, H, scale, 0.0, 0, window, 0,
                    -1.0);
 }
 

@@ -5,8 +5,10 @@
 //                    every row, rotates the shared key part and writes the
 //                    cache row.
 // latent_attention   for every (row, head): scores over the last `window`
-//                    positions, q_abs . c + rot(q_rot) . k_rot, softmax,
-//                    and the weighted sum of the latents c. The products
+//                    positions, q_abs . c + rot(q_rot) . k_rot, softmax
+//                    (in which a sink per head, a score without a latent, may
+//                    take part), and the weighted sum of the latents c. The
+//                    products
 //                    with the per-head key and value expansions live
 //                    outside, on the query and output side.
 //
@@ -109,6 +111,14 @@ void latent_kv_append(torch::Tensor cq_out, torch::Tensor cache,
   HIP_CHECK_KERNEL();
 }
 
+// What a sum over keys with maximum m and weight sum l is multiplied by, once a
+// score `sink` without a value has joined (-inf: none).
+DEV_INLINE float lat_fold(float m, float l, float sink) {
+  const float M = fmaxf(m, sink);
+  const float f = __expf(m - M);
+  return f / fmaf(f, l, __expf(sink - M));
+}
+
 // ---------------------------------------------------------------------------
 // Row-wise attention, any sizes, both formats. Block = (row, HB heads), 256
 // threads. Keys are taken 256 at a time: thread j scores key j for the HB
@@ -125,7 +135,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     int cs_rows, int dims, const int* __restrict__ positions,
     const int* __restrict__ row_seq, const int* __restrict__ block_table,
     int max_blocks, long rows, int H, int dn, int dr, int R, int BS,
-    int window, float scale) {
+    int window, float scale, const float* __restrict__ sinks) {
   extern __shared__ float sm[];
   const int KW = R + dr;
   float* sq = sm;                          // [HB][KW] query (latent | rot)
@@ -240,7 +250,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
   for (int hb = 0; hb < LAT_HB; ++hb) {
     const int h = h0 + hb;
     if (h >= H) break;
-    const float inv = 1.0f / l[hb];
+    const float inv = lat_fold(m[hb], l[hb], sinks ? sinks[h] : -INFINITY);
 #pragma unroll
     for (int k = 0; k < ND; ++k) {
       const int d = tid + k * 256;
@@ -261,8 +271,8 @@ __global__ __launch_bounds__(256) void latent_attention_vec_kernel(
     int cs_rows, int dims, const int* __restrict__ positions,
     const int* __restrict__ row_seq, const int* __restrict__ block_table,
     int max_blocks, long rows, int H, int dn, int dr, int R, int BS,
-    int window, float scale, int NS, float* __restrict__ split_o,
-    float* __restrict__ split_ml) {
+    int window, float scale, const float* __restrict__ sinks, int NS,
+    float* __restrict__ split_o, float* __restrict__ split_ml) {
   extern __shared__ float sm[];
   const int KW = R + dr;
   float* sq = sm;                          // [HB][KW]
@@ -416,7 +426,8 @@ __global__ __launch_bounds__(256) void latent_attention_vec_kernel(
       mh = hb == x ? m[x] : mh;
     }
     if (NS == 1) {
-      stf(out + ((long)h * rows + r) * R + d, sum / lh);
+      stf(out + ((long)h * rows + r) * R + d,
+          sum * lat_fold(mh, lh, sinks ? sinks[h] : -INFINITY));
     } else {
       const long u = (r * H + h) * NS + blockIdx.z;
       split_o[u * R + d] = sum;
@@ -429,11 +440,13 @@ __global__ __launch_bounds__(256) void latent_attention_vec_kernel(
 }
 
 // Folds the key splits of a row: out = sum_z e^(m_z - M) o_z / sum_z
-// e^(m_z - M) l_z, splits in order. A row without keys gives zeros.
+// e^(m_z - M) l_z, splits in order, the sink last. A row without keys gives
+// zeros.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_attention_merge_kernel(
     T* __restrict__ out, const float* __restrict__ split_o,
-    const float* __restrict__ split_ml, long rows, int H, int R, int NS) {
+    const float* __restrict__ split_ml, const float* __restrict__ sinks,
+    long rows, int H, int R, int NS) {
   const long r = blockIdx.x;
   const int h = blockIdx.y;
   const long u0 = (r * H + h) * NS;
@@ -444,13 +457,15 @@ __global__ __launch_bounds__(256) void latent_attention_merge_kernel(
     const float mz = split_ml[(u0 + z) * 2];
     if (mz > -INFINITY) L += __expf(mz - M) * split_ml[(u0 + z) * 2 + 1];
   }
+  const float f =
+      L > 0.f ? lat_fold(M, L, sinks ? sinks[h] : -INFINITY) : 0.f;
   for (int d = threadIdx.x; d < R; d += blockDim.x) {
     float acc = 0.f;
     for (int z = 0; z < NS; ++z) {
       const float mz = split_ml[(u0 + z) * 2];
       if (mz > -INFINITY) acc += __expf(mz - M) * split_o[(u0 + z) * R + d];
     }
-    stf(out + ((long)h * rows + r) * R + d, L > 0.f ? acc / L : 0.f);
+    stf(out + ((long)h * rows + r) * R + d, acc * f);
   }
 }
 
@@ -491,8 +506,9 @@ __global__ __launch_bounds__(128) void latent_attention_mfma_kernel(
     const float* __restrict__ cs, int cs_rows, int dims,
     const int* __restrict__ positions, const int* __restrict__ row_seq,
     const int* __restrict__ block_table, int max_blocks, long rows, int H,
-    int dn, int BS, int window, float scale, int HT, int NS,
-    float* __restrict__ split_o, float* __restrict__ split_ml) {
+    int dn, int BS, int window, float scale, const float* __restrict__ sinks,
+    int HT, int NS, float* __restrict__ split_o,
+    float* __restrict__ split_ml) {
   constexpr int KW = R + DR, KST = KW / 32, VST = R / 32, NDT = R / 16;
   constexpr int LDV = R + 8;               // padded LDS row, 16-byte aligned
   extern __shared__ unsigned short lat_lds[];
@@ -639,7 +655,7 @@ __global__ __launch_bounds__(128) void latent_attention_mfma_kernel(
     }
     return;
   }
-  const float inv = 1.0f / l;
+  const float inv = lat_fold(m, l, sinks ? sinks[h] : -INFINITY);
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt) {
     const unsigned int w0 = (unsigned int)f2us(o[dt][0] * inv) |
@@ -657,7 +673,7 @@ static void launch_latent_mfma(torch::Tensor& out, torch::Tensor& q_abs,
                                torch::Tensor& row_seq,
                                torch::Tensor& block_table, long rows, int H,
                                int dn, int window, float scale,
-                               hipStream_t stream) {
+                               const float* sinks, hipStream_t stream) {
   const int HT = (H + 15) / 16;
   const long units = rows * HT;
   const size_t lds = (size_t)2 * 16 * (R + 8) * sizeof(unsigned short);
@@ -682,14 +698,14 @@ static void launch_latent_mfma(torch::Tensor& out, torch::Tensor& q_abs,
           cs.data_ptr<float>(), (int)cs.size(0), (int)cs.size(1),
           positions.data_ptr<int>(), row_seq.data_ptr<int>(),
           block_table.data_ptr<int>(), (int)block_table.size(1), rows, H, dn,
-          (int)cache.size(2), window, scale, HT, NS,
+          (int)cache.size(2), window, scale, sinks, HT, NS,
           NS > 1 ? so.data_ptr<float>() : nullptr,
           NS > 1 ? sml.data_ptr<float>() : nullptr);
   if (NS > 1)
     latent_attention_merge_kernel<bf16_t>
         <<<dim3((unsigned)rows, (unsigned)H), 256, 0, stream>>>(
             reinterpret_cast<bf16_t*>(out.data_ptr()), so.data_ptr<float>(),
-            sml.data_ptr<float>(), rows, H, R, NS);
+            sml.data_ptr<float>(), sinks, rows, H, R, NS);
 }
 
 // sizes the matrix-core form serves
@@ -698,12 +714,14 @@ bool latent_attention_mfma_supported(int64_t R, int64_t dr) {
 }
 
 // out, q_abs [H, rows, R] contiguous; q [rows, >= H*(dn+dr)] (stride(1) ==
-// 1); cache [blocks, 1, BS, R+dr]; cs [positions, dims] fp32.
+// 1); cache [blocks, 1, BS, R+dr]; cs [positions, dims] fp32; sinks [H] fp32 or
+// empty.
 void latent_attention(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q,
                       torch::Tensor cache, torch::Tensor cs,
                       torch::Tensor positions, torch::Tensor row_seq,
                       torch::Tensor block_table, int64_t H, int64_t dn,
-                      int64_t dr, int64_t window, double scale) {
+                      int64_t dr, int64_t window, double scale,
+                      torch::Tensor sinks) {
   check_act(q, "q"); check_act(q_abs, "q_abs"); check_act(out, "out");
   check_f32(cs, "cs");
   check_i32(positions, "positions"); check_i32(row_seq, "row_seq");
@@ -725,6 +743,12 @@ void latent_attention(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q,
               cs.size(1) <= dr);
   TORCH_CHECK(positions.numel() == rows && row_seq.numel() == rows);
   TORCH_CHECK(block_table.dim() == 2);
+  const float* sp = nullptr;
+  if (sinks.numel() > 0) {
+    check_f32(sinks, "sinks");
+    TORCH_CHECK(sinks.numel() == H);
+    sp = sinks.data_ptr<float>();
+  }
   TORCH_CHECK(R <= 1024, "latent_attention: latent wider than 1024");
   if (rows == 0) return;
   const size_t lds = (size_t)(LAT_HB * (R + dr) + LAT_HB * LAT_CH) * 4;
@@ -740,7 +764,7 @@ void latent_attention(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q,
 #define KK_MFMA(RR, DD)                                                      \
   launch_latent_mfma<RR, DD>(out, q_abs, q, cache, cs, positions, row_seq,   \
                              block_table, rows, (int)H, (int)dn, (int)window, \
-                             (float)scale, stream)
+                             (float)scale, sp, stream)
     if (R == 128 && dr == 32) KK_MFMA(128, 32);
     else if (R == 128) KK_MFMA(128, 64);
     else if (R == 256 && dr == 32) KK_MFMA(256, 32);
@@ -764,7 +788,7 @@ void latent_attention(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q,
         (int)cs.size(0), (int)cs.size(1), positions.data_ptr<int>(),         \
         row_seq.data_ptr<int>(), block_table.data_ptr<int>(),                \
         (int)block_table.size(1), rows, (int)H, (int)dn, (int)dr, R,         \
-        (int)cache.size(2), (int)window, (float)scale
+        (int)cache.size(2), (int)window, (float)scale, sp
   KK_DISPATCH_ACT(q, {
     if (vec && lds_vec <= 60 * 1024) {
       // few rows: split every row's keys over several workgroups
@@ -787,7 +811,7 @@ void latent_attention(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q,
         latent_attention_merge_kernel<T>
             <<<dim3((unsigned)rows, (unsigned)H), 256, 0, stream>>>(
                 reinterpret_cast<T*>(out.data_ptr()), so.data_ptr<float>(),
-                sml.data_ptr<float>(), rows, (int)H, R, NS);
+                sml.data_ptr<float>(), sp, rows, (int)H, R, NS);
       }
     } else if (R <= 256)
       latent_attention_kernel<T, 1><<<grid, 256, lds, stream>>>(KK_ARGS);

@@ -127,13 +127,14 @@ DEV_INLINE unsigned int cvt_pk_bf16(float lo, float hi) {
 // the first position of the query's chunk, scores pass cap * tanh(s / cap),
 // and the softmax weights enter the PV product as hi + lo (two bf16 terms)
 // so that they keep fp32-grade accuracy. EXT also serves a sliding window
-// (keys from q - window + 1 on) and a distance bias slope_h (q - k) taken off
-// head h's scores; with the key cache passed as the value cache too, the
-// values are the keys. EXT == 2 takes besides a logarithmic distance bias
+// (keys from q - window + 1 on, and positions below `keep`, whose tiles come
+// ahead of the window's), a distance bias slope_h (q - k) taken off head h's
+// scores, and a sink per head: the softmax starts from a score that has no
+// value. With the key cache passed as the value cache too, the values are the
+// keys. EXT == 2 takes besides a logarithmic distance bias
 // r1_h ln(1 + r2_h (q - k)) (a wave's 63 distances of a tile are one logarithm
-// per lane, handed over through LDS), keys divided by their own root mean
-// square (formed while the tile is staged), and a sink: the softmax starts from
-// a score of 0 that has no value.
+// per lane, handed over through LDS) and keys divided by their own root mean
+// square (formed while the tile is staged).
 template <int BS, bool FP8, int EXT>
 __global__ __launch_bounds__(256, EXT == 2 ? 2 : 1) void prefill_attn_kernel(
     unsigned short* __restrict__ out,       // [T, Hq*D]
@@ -148,7 +149,8 @@ __global__ __launch_bounds__(256, EXT == 2 ? 2 : 1) void prefill_attn_kernel(
     long q_stride, long q_offset, int Hq, int Hk, int max_blocks,
     int out_stride, float scale, float cap, int chunk, int window,
     const float* __restrict__ slopes, const float* __restrict__ r1,
-    const float* __restrict__ r2, float key_eps, int sink) {
+    const float* __restrict__ r2, float key_eps,
+    const float* __restrict__ sinks, int keep) {
   constexpr int D = 128;
   constexpr int KVT = 32;
   // 16-B aligned: staged via uint4 stores (guide G17)
@@ -202,14 +204,18 @@ __global__ __launch_bounds__(256, EXT == 2 ? 2 : 1) void prefill_attn_kernel(
   }
 
   float m = -INFINITY, l_acc = 0.f;
-  if (EXT == 2 && sink) { m = 0.f; l_acc = 1.f; }
+  if (EXT && sinks) { m = sinks[head]; l_acc = 1.f; }
   f32x16_t oacc[4] = {{}, {}, {}, {}};
 
   const int kv_limit = min(ctx, abs_start + qb0 + qn);
   const int ntiles = (kv_limit + KVT - 1) / KVT;
   const int nblocks = (ctx + BS - 1) / BS;
 
-  for (int ti = tile_lo / KVT; ti < ntiles; ++ti) {
+  // tiles of kept first tokens, then the ones from the first visible key on
+  const int tfirst = tile_lo / KVT;
+  const int nkept = EXT ? min(tfirst, (keep + KVT - 1) / KVT) : 0;
+  for (int it = 0; it < nkept + ntiles - tfirst; ++it) {
+    const int ti = it < nkept ? it : tfirst + it - nkept;
     const int kvbase = ti * KVT;
     // ---- cooperative stage ----
     {
@@ -329,7 +335,7 @@ __global__ __launch_bounds__(256, EXT == 2 ? 2 : 1) void prefill_attn_kernel(
       const int kvrow = (r & 3) + 8 * (r >> 2) + 4 * hi;
       const int kvpos = kvbase + kvrow;
       const bool valid = (kvpos <= q_abs) && (kvpos < ctx) &&
-                         (!EXT || kvpos >= q_lo);
+                         (!EXT || kvpos >= q_lo || kvpos < keep);
       float sc;
       if (EXT == 2) {
         sc = sacc[r] * kscale[kvrow];
@@ -469,7 +475,7 @@ void prefill_attention(torch::Tensor out, torch::Tensor q,
       seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),                    \
       qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0),         \
       q_offset, Hq, Hk, (int)block_table.size(1), (int)out.stride(0),        \
-      (float)scale, 0.f, 0, 0, nullptr, nullptr, nullptr, -1.f, 0)
+      (float)scale, 0.f, 0, 0, nullptr, nullptr, nullptr, -1.f, nullptr, 0)
   if (fp8) { PF_LAUNCH(true); } else { PF_LAUNCH(false); }
 #undef PF_LAUNCH
   HIP_CHECK_KERNEL();
@@ -522,7 +528,8 @@ void chunk_attention_tiles(torch::Tensor out, torch::Tensor q,
       seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),
       qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0), 0L, Hq,
       Hk, (int)block_table.size(1), (int)out.stride(0), (float)scale,
-      (float)softcap, (int)chunk, 0, nullptr, nullptr, nullptr, -1.f, 0);
+      (float)softcap, (int)chunk, 0, nullptr, nullptr, nullptr, -1.f, nullptr,
+      0);
   HIP_CHECK_KERNEL();
 }
 
@@ -576,23 +583,28 @@ void window_attention_tiles(torch::Tensor out, torch::Tensor q,
       qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0), 0L, Hq,
       Hk, (int)block_table.size(1), (int)out.stride(0), (float)scale, 0.f, 0,
       (int)window, biased ? slopes.data_ptr<float>() : nullptr, nullptr,
-      nullptr, -1.f, 0);
+      nullptr, -1.f, nullptr, 0);
   HIP_CHECK_KERNEL();
 }
 
-// Prompt portions of chunk-local attention over key-only pages (the values are
-// the keys) with capped scores, a logarithmic distance bias, keys divided by
-// their root mean square as they are read (key_eps >= 0) and a sink: out, q
-// [T, H*128] contiguous, k_cache [blocks, G, 16, 128], r1, r2 [H] fp32 or
-// empty.
+// Prompt portions of attention with the options of masked_attention on the
+// matrix cores: chunk, window with kept first tokens, capped scores, a
+// logarithmic distance bias, keys divided by their root mean square as they are
+// read (key_eps >= 0), sinks. out, q [T, H*128] contiguous, k_cache [blocks, G,
+// 16, 128], v_cache the same or empty (the values are the keys), r1, r2, sinks
+// [H] fp32 or empty.
 void masked_attention_tiles(torch::Tensor out, torch::Tensor q,
-                            torch::Tensor k_cache, torch::Tensor r1,
-                            torch::Tensor r2, torch::Tensor block_table,
+                            torch::Tensor k_cache, torch::Tensor v_cache,
+                            torch::Tensor r1, torch::Tensor r2,
+                            torch::Tensor sinks, torch::Tensor block_table,
                             torch::Tensor seq_lens, torch::Tensor q_starts,
                             torch::Tensor qb_seq, torch::Tensor qb_start,
                             double scale, double softcap, int64_t chunk,
-                            bool sink, double key_eps) {
+                            int64_t window, int64_t keep, double key_eps) {
   TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous());
+  if (v_cache.numel() == 0) v_cache = k_cache;
+  TORCH_CHECK(v_cache.sizes() == k_cache.sizes() && v_cache.is_contiguous() &&
+              v_cache.scalar_type() == k_cache.scalar_type());
   const int Hk = (int)k_cache.size(1);
   TORCH_CHECK(window_attention_tiles_supported(k_cache.size(3),
                                                k_cache.size(2)));
@@ -604,11 +616,14 @@ void masked_attention_tiles(torch::Tensor out, torch::Tensor q,
               out.size(1) == q.size(1) && q.size(1) % 128 == 0);
   const int Hq = (int)(q.size(1) / 128);
   TORCH_CHECK(Hq % Hk == 0 && chunk >= 0);
-  const bool logb = r1.numel() > 0;
-  if (logb)
-    for (const auto& t : {r1, r2})
-      TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 &&
-                  t.is_contiguous() && t.numel() == Hq);
+  TORCH_CHECK(window >= 0 && keep >= 0);
+  const bool logb = r1.numel() > 0, sunk = sinks.numel() > 0;
+  const auto per_head = [&](const torch::Tensor& t) {
+    return t.is_cuda() && t.scalar_type() == torch::kFloat32 &&
+           t.is_contiguous() && t.numel() == Hq;
+  };
+  TORCH_CHECK(!logb || (per_head(r1) && per_head(r2)));
+  TORCH_CHECK(!sunk || per_head(sinks));
   TORCH_CHECK(q_starts.dim() == 2 && q_starts.size(1) == 2);
   TORCH_CHECK(qb_seq.scalar_type() == torch::kInt32 &&
               qb_start.scalar_type() == torch::kInt32 &&
@@ -620,16 +635,21 @@ void masked_attention_tiles(torch::Tensor out, torch::Tensor q,
   const int G = Hq / Hk;
   auto stream = c10::hip::getCurrentHIPStream().stream();
   dim3 grid(nqb, Hk, (G + 3) / 4);
-  prefill_attn_kernel<16, false, 2><<<grid, 256, 0, stream>>>(
-      reinterpret_cast<unsigned short*>(out.data_ptr()),
-      reinterpret_cast<const unsigned short*>(q.data_ptr()),
-      k_cache.data_ptr(), k_cache.data_ptr(), block_table.data_ptr<int>(),
-      seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),
-      qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0), 0L, Hq,
-      Hk, (int)block_table.size(1), (int)out.stride(0), (float)scale,
-      (float)softcap, (int)chunk, 0, nullptr,
-      logb ? r1.data_ptr<float>() : nullptr,
-      logb ? r2.data_ptr<float>() : nullptr, (float)key_eps, (int)sink);
+#define KK_LAUNCH(EXT_)                                                      \
+  prefill_attn_kernel<16, false, EXT_><<<grid, 256, 0, stream>>>(            \
+      reinterpret_cast<unsigned short*>(out.data_ptr()),                     \
+      reinterpret_cast<const unsigned short*>(q.data_ptr()),                 \
+      k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr<int>(),   \
+      seq_lens.data_ptr<int>(), q_starts.data_ptr<int>(),                    \
+      qb_seq.data_ptr<int>(), qb_start.data_ptr<int>(), q.stride(0), 0L, Hq, \
+      Hk, (int)block_table.size(1), (int)out.stride(0), (float)scale,        \
+      (float)softcap, (int)chunk, (int)window, nullptr,                      \
+      logb ? r1.data_ptr<float>() : nullptr,                                 \
+      logb ? r2.data_ptr<float>() : nullptr, (float)key_eps,                 \
+      sunk ? sinks.data_ptr<float>() : nullptr, (int)keep)
+  // the log bias and the key norm take the second form
+  if (logb || key_eps >= 0) { KK_LAUNCH(2); } else { KK_LAUNCH(1); }
+#undef KK_LAUNCH
   HIP_CHECK_KERNEL();
 }
 

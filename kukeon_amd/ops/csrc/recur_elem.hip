@@ -1,7 +1,8 @@
 // Small per-row and per-element kernels of the recurrent / latent group:
 //   gated_group_rmsnorm  out = rmsnorm_by_part(y * silu(z)) * w
 //   head_gate            out[t, h, :] = o[h, t, :] * sigmoid(gate[t, h]), or
-//                        entry by entry with a gate of H*dv columns
+//                        entry by entry with a gate of H*dv columns, or the
+//                        heads merely brought together without a gate
 //   xielu                piecewise quadratic / exponential activation
 //   softcap_             logits <- cap * tanh(logits / cap)
 #include "elem.h"
@@ -124,7 +125,7 @@ void gated_group_rmsnorm(torch::Tensor out, torch::Tensor y, torch::Tensor z,
   HIP_CHECK_KERNEL();
 }
 
-// gw: gate columns per head (1: one gate per head, dv: one per entry)
+// gw: gate columns per head (0: no gate, 1: one per head, dv: one per entry)
 template <typename T>
 __global__ __launch_bounds__(256) void head_gate_kernel(
     T* __restrict__ out, const T* __restrict__ o, const T* __restrict__ gate,
@@ -136,7 +137,8 @@ __global__ __launch_bounds__(256) void head_gate_kernel(
   const int h = (int)((i / dv) % H);
   const long t = i / ((long)dv * H);
   const long gc = gw == 1 ? h : (long)h * dv + d;
-  const float g = 1.0f / (1.0f + __expf(-ldf(gate + t * ldg + gc)));
+  const float g =
+      gw == 0 ? 1.0f : 1.0f / (1.0f + __expf(-ldf(gate + t * ldg + gc)));
   stf(out + i, ldf(o + ((long)h * rows + t) * dv + d) * g);
 }
 
@@ -157,7 +159,7 @@ __global__ __launch_bounds__(256) void head_gate_vec_kernel(
     const float g = 1.0f / (1.0f + __expf(-ldf(gate + t * ldg + h)));
 #pragma unroll
     for (int k = 0; k < 8; ++k) v[k] *= g;
-  } else {
+  } else if (gw > 1) {
     float g[8];
     ld8(gate + t * ldg + (long)h * dv + d, g);
 #pragma unroll
@@ -167,29 +169,30 @@ __global__ __launch_bounds__(256) void head_gate_vec_kernel(
 }
 
 // out [T, H*dv]; o [H, T, dv] contiguous; gate [T, H] or [T, H*dv] (any row
-// stride).
+// stride), or empty.
 void head_gate(torch::Tensor out, torch::Tensor o, torch::Tensor gate) {
   check_act(out, "out"); check_act(o, "o"); check_act(gate, "gate");
   TORCH_CHECK(o.dim() == 3 && o.is_contiguous() && out.is_contiguous());
   const long H = o.size(0), rows = o.size(1), dv = o.size(2);
   TORCH_CHECK(out.dim() == 2 && out.size(0) == rows && out.size(1) == H * dv);
-  TORCH_CHECK(gate.dim() == 2 && gate.size(0) == rows &&
-              (gate.size(1) == H || gate.size(1) == H * dv) &&
-              gate.stride(1) == 1);
-  const int gw = gate.size(1) == H ? 1 : (int)dv;
+  const bool gated = gate.numel() > 0;
+  TORCH_CHECK(!gated || (gate.dim() == 2 && gate.size(0) == rows &&
+                         (gate.size(1) == H || gate.size(1) == H * dv) &&
+                         gate.stride(1) == 1));
+  const int gw = !gated ? 0 : gate.size(1) == H ? 1 : (int)dv;
   TORCH_CHECK(o.scalar_type() == out.scalar_type() &&
               gate.scalar_type() == out.scalar_type());
   const long total = rows * H * dv;
   if (total == 0) return;
   auto stream = c10::hip::getCurrentHIPStream().stream();
   if (dv % 8 == 0 && aligned16(out.data_ptr()) && aligned16(o.data_ptr()) &&
-      (gw == 1 || (gate.stride(0) % 8 == 0 && aligned16(gate.data_ptr())))) {
+      (gw <= 1 || (gate.stride(0) % 8 == 0 && aligned16(gate.data_ptr())))) {
     KK_DISPATCH_ACT(out, {
       head_gate_vec_kernel<T><<<dim3((unsigned)((total / 8 + 255) / 256)), 256,
                                 0, stream>>>(
           reinterpret_cast<T*>(out.data_ptr()),
           reinterpret_cast<const T*>(o.data_ptr()),
-          reinterpret_cast<const T*>(gate.data_ptr()), (long)gate.stride(0),
+          reinterpret_cast<const T*>(gate.data_ptr()), gated ? (long)gate.stride(0) : 0L,
           rows, (int)H, (int)dv, gw);
     });
     HIP_CHECK_KERNEL();
@@ -200,7 +203,7 @@ void head_gate(torch::Tensor out, torch::Tensor o, torch::Tensor gate) {
                           stream>>>(
         reinterpret_cast<T*>(out.data_ptr()),
         reinterpret_cast<const T*>(o.data_ptr()),
-        reinterpret_cast<const T*>(gate.data_ptr()), (long)gate.stride(0),
+        reinterpret_cast<const T*>(gate.data_ptr()), gated ? (long)gate.stride(0) : 0L,
         rows, (int)H, (int)dv, gw);
   });
   HIP_CHECK_KERNEL();

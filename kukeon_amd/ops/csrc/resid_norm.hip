@@ -1,7 +1,8 @@
 // Residual stream kept in fp32: x += a (+ bias), then h = rmsnorm(x) with a
 // weight stored as an offset from a constant (weight_offset + w). One block
 // per row; the row's sum of squares is reduced in a fixed order, so a row's
-// result does not depend on what else is in the batch.
+// result does not depend on what else is in the batch. Also the start of a stack
+// whose embedding rows are normed: x = rmsnorm(table[id]), h = rmsnorm(x).
 #include "elem.h"
 
 namespace kukeon {
@@ -142,6 +143,119 @@ void residual_add_rmsnorm(torch::Tensor x, torch::Tensor a, torch::Tensor bias,
         has_b ? bias.data_ptr<float>() : nullptr, w.data_ptr<float>(),
         (float)w_offset, (float)eps, reinterpret_cast<T*>(out.data_ptr()), W);
   });
+  HIP_CHECK_KERNEL();
+}
+
+// x = rmsnorm(table[id]) * (w_offset + w), out = rmsnorm(x) * (w_offset + w2).
+// One block per row; NIT > 0: W a multiple of 8 and at most 8 * 256 * NIT, the
+// row held in registers; NIT == 0: any width.
+template <typename T, int NIT>
+__global__ __launch_bounds__(256) void embed_rmsnorm_kernel(
+    float* __restrict__ x, T* __restrict__ out, const int* __restrict__ ids,
+    const T* __restrict__ table, long vocab, const float* __restrict__ w,
+    const float* __restrict__ w2, float w_offset, float eps, int W) {
+  __shared__ float red[32];
+  const long row = blockIdx.x;
+  const long id = min(max((long)ids[row], 0L), vocab - 1);
+  const T* er = table + id * W;
+  float* xr = x + row * (long)W;
+  T* orow = out + row * (long)W;
+  if (NIT > 0) {
+    float v[NIT > 0 ? NIT : 1][8];
+    float ss = 0.f;
+#pragma unroll
+    for (int it = 0; it < NIT; ++it) {
+      const int i = (it * 256 + threadIdx.x) * 8;
+      if (i < W) {
+        ld8(er + i, v[it]);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) ss += v[it][k] * v[it][k];
+      }
+    }
+    const float2 t1 = block_sum2(ss, 0.f, red);
+    const float re = 1.0f / sqrtf(t1.x / (float)W + eps);
+    float sx = 0.f;
+#pragma unroll
+    for (int it = 0; it < NIT; ++it) {
+      const int i = (it * 256 + threadIdx.x) * 8;
+      if (i < W) {
+        float t[8];
+        ld8(w + i, t);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {
+          v[it][k] = v[it][k] * re * (w_offset + t[k]);
+          sx += v[it][k] * v[it][k];
+        }
+        st8(xr + i, v[it]);
+      }
+    }
+    const float2 t2 = block_sum2(sx, 0.f, red);
+    const float rx = 1.0f / sqrtf(t2.x / (float)W + eps);
+#pragma unroll
+    for (int it = 0; it < NIT; ++it) {
+      const int i = (it * 256 + threadIdx.x) * 8;
+      if (i < W) {
+        float t[8], o[8];
+        ld8(w2 + i, t);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) o[k] = v[it][k] * rx * (w_offset + t[k]);
+        st8(orow + i, o);
+      }
+    }
+    return;
+  }
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float v = ldf(er + i);
+    ss += v * v;
+  }
+  const float2 t1 = block_sum2(ss, 0.f, red);
+  const float re = 1.0f / sqrtf(t1.x / (float)W + eps);
+  float sx = 0.f;
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float v = ldf(er + i) * re * (w_offset + w[i]);
+    xr[i] = v;
+    sx += v * v;
+  }
+  const float2 t2 = block_sum2(sx, 0.f, red);
+  const float rx = 1.0f / sqrtf(t2.x / (float)W + eps);
+  for (int i = threadIdx.x; i < W; i += blockDim.x)
+    stf(orow + i, xr[i] * rx * (w_offset + w2[i]));
+}
+
+// x [T, W] fp32; out [T, W] and table [vocab, W] in the activation format; ids
+// [T] int32 (kept within the table); w, w2 [W] fp32.
+void embed_rmsnorm(torch::Tensor x, torch::Tensor out, torch::Tensor ids,
+                   torch::Tensor table, torch::Tensor w, torch::Tensor w2,
+                   double w_offset, double eps) {
+  check_f32(x, "x"); check_f32(w, "w"); check_f32(w2, "w2");
+  check_act(out, "out"); check_act(table, "table"); check_i32(ids, "ids");
+  TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && out.is_contiguous() &&
+              out.sizes() == x.sizes());
+  const long rows = x.size(0);
+  const int W = (int)x.size(1);
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && table.size(1) == W &&
+              table.size(0) >= 1 && table.scalar_type() == out.scalar_type());
+  TORCH_CHECK(ids.numel() == rows && w.numel() == W && w2.numel() == W);
+  if (rows == 0) return;
+  auto stream = c10::hip::getCurrentHIPStream().stream();
+  const bool vec = W % 8 == 0 && W <= 8 * 256 * 4 && aligned16(x.data_ptr()) &&
+                   aligned16(out.data_ptr()) && aligned16(table.data_ptr()) &&
+                   aligned16(w.data_ptr()) && aligned16(w2.data_ptr());
+  dim3 grid((unsigned)rows);
+#define KK_ARGS x.data_ptr<float>(), reinterpret_cast<T*>(out.data_ptr()),     \
+        ids.data_ptr<int>(), reinterpret_cast<const T*>(table.data_ptr()),     \
+        (long)table.size(0), w.data_ptr<float>(), w2.data_ptr<float>(),        \
+        (float)w_offset, (float)eps, W
+  KK_DISPATCH_ACT(out, {
+    if (!vec) embed_rmsnorm_kernel<T, 0><<<grid, 256, 0, stream>>>(KK_ARGS);
+    else if (W <= 2048)
+      embed_rmsnorm_kernel<T, 1><<<grid, 256, 0, stream>>>(KK_ARGS);
+    else if (W <= 4096)
+      embed_rmsnorm_kernel<T, 2><<<grid, 256, 0, stream>>>(KK_ARGS);
+    else embed_rmsnorm_kernel<T, 4><<<grid, 256, 0, stream>>>(KK_ARGS);
+  });
+#undef KK_ARGS
   HIP_CHECK_KERNEL();
 }
 

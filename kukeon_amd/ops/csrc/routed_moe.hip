@@ -7,6 +7,11 @@
 //                          chosen scores are divided by their sum and scaled
 //   router_sigmoid         scores = sigmoid of every logit by itself; the `top`
 //                          largest, as they are, times a scale
+//   router_corrected       scores = sigmoid of every logit; the choice goes by
+//                          score plus a learned correction per expert, within
+//                          the best runs of neighbours (by the sum of a run's
+//                          largest few choice scores); the weights are the
+//                          scores without it, divided by their sum if asked
 //   combine_rows_weighted  out[t] = sum_k w[t, k] * in[inv[t, k]], the k-th
 //                          term added k-th, fp32 sums
 // The expert GEMMs themselves are vendor GEMMs over gathered rows.
@@ -223,6 +228,124 @@ void router_sigmoid(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
       idx.data_ptr<int>(), wts.data_ptr<float>(), (long)idx.stride(0),
       (long)wts.stride(0), logits.data_ptr<float>(), (long)logits.stride(0),
       rows, E, (int)top, (float)scale);
+  HIP_CHECK_KERNEL();
+}
+
+// The largest (value, -index) pair of a wave; every lane gets the index.
+DEV_INLINE int wave_argmax(float v, int i) {
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) {
+    const float ov = __shfl_xor(v, off, WAVE);
+    const int oi = __shfl_xor(i, off, WAVE);
+    if (ov > v || (ov == v && oi < i)) { v = ov; i = oi; }
+  }
+  return i;
+}
+
+// One wave per row, experts over the lanes. In LDS: scores s [E], choice
+// scores c [E], run scores [groups]. -inf marks what cannot be chosen (any
+// more); a NaN logit counts as a score of 0 and the lowest choice score.
+__global__ __launch_bounds__(64) void router_corrected_kernel(
+    int* __restrict__ idx, float* __restrict__ wts, long ldi, long ldw,
+    const float* __restrict__ logits, long ldz,
+    const float* __restrict__ correction, int E, int top, int groups, int keep,
+    int best, float scale, int renorm) {
+  extern __shared__ float sm[];
+  float* s = sm;
+  float* c = s + E;
+  float* gs = c + E;
+  const long t = blockIdx.x;
+  const int lane = threadIdx.x;
+  const float* z = logits + t * ldz;
+  for (int e = lane; e < E; e += WAVE) {
+    const float sc = 1.0f / (1.0f + expf(-z[e]));
+    const float ch = correction ? sc + correction[e] : sc;
+    s[e] = sc == sc ? sc : 0.f;
+    c[e] = ch == ch ? fmaxf(ch, -3.0e38f) : -3.0e38f;
+  }
+  __syncthreads();
+  if (groups > 0) {
+    const int per = E / groups;
+    for (int g = lane; g < groups; g += WAVE) {
+      float a = -INFINITY, b = -INFINITY;       // the two largest
+      for (int e = g * per; e < (g + 1) * per; ++e) {
+        const float v = c[e];
+        b = fmaxf(b, fminf(a, v));
+        a = fmaxf(a, v);
+      }
+      gs[g] = fmaxf(best > 1 && per > 1 ? a + b : a, -3.0e38f);
+    }
+    __syncthreads();
+    for (int k = 0; k < keep; ++k) {
+      float v = -INFINITY;
+      int i = groups;
+      for (int g = lane; g < groups; g += WAVE)
+        if (gs[g] > v) { v = gs[g]; i = g; }
+      i = min(wave_argmax(v, i), groups - 1);
+      __syncthreads();
+      if (lane == 0) gs[i] = -INFINITY;         // taken
+      __syncthreads();
+    }
+    for (int e = lane; e < E; e += WAVE)
+      if (gs[e / per] != -INFINITY) c[e] = -INFINITY;
+    __syncthreads();
+  }
+  float sum = 0.f;
+  for (int k = 0; k < top; ++k) {
+    float v = -INFINITY;
+    int i = E;
+    for (int e = lane; e < E; e += WAVE)
+      if (c[e] > v) { v = c[e]; i = e; }
+    i = min(wave_argmax(v, i), E - 1);
+    sum += s[i];
+    if (lane == 0) idx[t * ldi + k] = i;
+    if (lane == (k & (WAVE - 1))) wts[t * ldw + k] = s[i];
+    __syncthreads();
+    if (lane == 0) c[i] = -INFINITY;
+    __syncthreads();
+  }
+  const float f = renorm ? scale / (sum + 1e-20f) : scale;
+  // lane k & 63 wrote weight k and reads it back
+  for (int k = lane; k < top; k += WAVE) wts[t * ldw + k] *= f;
+}
+
+// idx [T, >= top] int32, wts [T, >= top] fp32, logits [T, E] fp32 (row strides
+// free); correction [E] fp32 or empty; groups 0: every expert can be chosen;
+// best: how many of a run's largest choice scores make its own (1 or 2).
+void router_corrected(torch::Tensor idx, torch::Tensor wts,
+                      torch::Tensor logits, torch::Tensor correction,
+                      int64_t top, int64_t groups, int64_t keep, int64_t best,
+                      double scale, bool renorm) {
+  TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == torch::kFloat32 &&
+              logits.dim() == 2 && logits.stride(1) == 1,
+              "logits must be fp32 rows");
+  TORCH_CHECK(idx.is_cuda() && idx.scalar_type() == torch::kInt32 &&
+              wts.is_cuda() && wts.scalar_type() == torch::kFloat32);
+  TORCH_CHECK(idx.dim() == 2 && wts.dim() == 2);
+  const long rows = logits.size(0);
+  const int E = (int)logits.size(1);
+  TORCH_CHECK(top >= 1 && top <= E && (best == 1 || best == 2));
+  TORCH_CHECK(idx.size(0) == rows && wts.size(0) == rows &&
+              idx.size(1) >= top && wts.size(1) >= top &&
+              idx.stride(1) == 1 && wts.stride(1) == 1);
+  TORCH_CHECK(groups >= 0 && groups <= E);
+  if (groups > 0)
+    TORCH_CHECK(E % groups == 0 && keep >= 1 && keep <= groups &&
+                top <= keep * (E / groups));
+  const bool corr = correction.numel() > 0;
+  if (corr) {
+    check_f32(correction, "correction");
+    TORCH_CHECK(correction.numel() == E);
+  }
+  const size_t lds = (size_t)(2 * E + groups) * sizeof(float);
+  TORCH_CHECK(lds <= 60 * 1024, "router_corrected: too many experts");
+  if (rows == 0) return;
+  auto stream = c10::hip::getCurrentHIPStream().stream();
+  router_corrected_kernel<<<dim3((unsigned)rows), 64, lds, stream>>>(
+      idx.data_ptr<int>(), wts.data_ptr<float>(), (long)idx.stride(0),
+      (long)wts.stride(0), logits.data_ptr<float>(), (long)logits.stride(0),
+      corr ? correction.data_ptr<float>() : nullptr, E, (int)top, (int)groups,
+      (int)keep, (int)best, (float)scale, (int)renorm);
   HIP_CHECK_KERNEL();
 }
 

@@ -521,13 +521,14 @@ def latent_kv_append(cq_out, cache, proj, q_col: int, kv_col: int, wq, wkv,
 
 def latent_attention(out, q_abs, q, cache, cs, positions, row_seq,
                      block_table, H: int, dn: int, dr: int, window: int,
-                     scale: float) -> None:
+                     scale: float, sinks) -> None:
     """Attention of H heads over ONE shared cache row per token,
     [latent (R) | rotated key part (dr)]. q_abs [H, T, R] is the query
     already multiplied into latent space; q [T, H*(dn+dr)] holds the
     unrotated rotary part of every head behind its first dn entries.
     out [H, T, R] = softmax-weighted sum of the latents over the last
-    `window` positions."""
+    `window` positions; sinks [H] (or empty) join the softmax without a
+    latent."""
     R = q_abs.shape[2]
     BS = cache.shape[2]
     dims = cs.shape[1]
@@ -545,14 +546,19 @@ def latent_attention(out, q_abs, q, cache, cs, positions, row_seq,
         qr = _rot_pairs(q[r, : H * (dn + dr)].float().view(H, dn + dr)[:, dn:], cs[p], dims)
         sc = (q_abs[:, r].float() @ rows[:, :R].T +
               qr @ rows[:, R:].T) * scale                    # [H, n]
-        w = torch.softmax(sc, -1)
+        if sinks.numel():
+            sc = torch.cat([sc, sinks[:, None]], -1)
+        w = torch.softmax(sc, -1)[:, : len(js)]
         out[:, r] = (w @ rows[:, :R]).to(out.dtype)
 
 
 def head_gate(out, o, gate) -> None:
     """out[t, h*dv:(h+1)*dv] = o[h, t] * sigmoid(gate[t, h]); a gate with
-    H*dv columns acts entry by entry."""
+    H*dv columns acts entry by entry, an empty one not at all."""
     Hh, T, dv = o.shape
+    if not gate.numel():
+        out.copy_(o.permute(1, 0, 2).reshape(T, Hh * dv))
+        return
     g = torch.sigmoid(gate.float())                  # [T, H] or [T, H*dv]
     g = g.view(T, Hh, -1)                            # per head or per entry
     out.copy_((o.float().permute(1, 0, 2) * g).reshape(
@@ -1082,9 +1088,9 @@ def head_norm_append(q_out, k_cache, proj, q_col: int, k_col: int, w,
         k_cache[blk, :, p % BS] = proj[r, k_col: k_col + G * d].view(G, d)
 
 
-def masked_attention(out, q, k_cache, v_cache, slopes, r1, r2, positions,
-                     row_seq, block_table, H: int, scale: float,
-                     softcap: float, chunk: int, window: int, sink: bool,
+def masked_attention(out, q, k_cache, v_cache, slopes, r1, r2, sinks,
+                     positions, row_seq, block_table, H: int, scale: float,
+                     softcap: float, chunk: int, window: int, keep: int,
                      key_eps: float) -> None:
     G, BS, d = k_cache.shape[1], k_cache.shape[2], k_cache.shape[3]
     own_v = v_cache is not None and v_cache.numel() > 0
@@ -1098,7 +1104,8 @@ def masked_attention(out, q, k_cache, v_cache, slopes, r1, r2, positions,
         lo = p // chunk * chunk if chunk > 0 else 0
         if window > 0:
             lo = max(lo, p - window + 1)
-        js = torch.arange(lo, p + 1)
+        js = torch.cat([torch.arange(min(keep, lo)),
+                        torch.arange(lo, p + 1)])
         blk = block_table[s, (js // BS).long()].long()
         k = k_cache[blk, :, (js % BS).long()].float()         # [n, G, d]
         v = v_cache[blk, :, (js % BS).long()].float() if own_v else k
@@ -1115,8 +1122,8 @@ def masked_attention(out, q, k_cache, v_cache, slopes, r1, r2, positions,
                 sc = sc - slopes[h] * dist
             if r1.numel():
                 sc = sc - r1[h] * torch.log1p(r2[h] * dist)
-            if sink:
-                sc = torch.cat([sc, torch.zeros(1)])
+            if sinks.numel():
+                sc = torch.cat([sc, sinks[h: h + 1]])
                 w = torch.softmax(sc, -1)[:-1]
             else:
                 w = torch.softmax(sc, -1)
@@ -1154,3 +1161,56 @@ def routed_experts(out, h, idx, wts, top: int, w_gu, w_down, limit: float,
         if extra.numel():
             acc = acc + extra[t].float()
         out[t] = acc.to(out.dtype)
+
+
+# ---- sink group ------------------------------------------------------------
+def embed_rmsnorm(x, out, ids, table, w, w2, w_offset: float,
+                  eps: float) -> None:
+    rows = table[ids.long().clamp(0, table.shape[0] - 1)].float()
+    x.copy_(_unit_rms(rows, eps) * (w_offset + w))
+    out.copy_((_unit_rms(x, eps) * (w_offset + w2)).to(out.dtype))
+
+
+def rotary_append(q_out, k_cache, v_cache, proj, q_col: int, k_col: int,
+                  v_col: int, cs, positions, row_seq, block_table) -> None:
+    """Queries and keys rotated as pairs (2i, 2i+1) in their first
+    cs.shape[1] entries; key and value rows to their page."""
+    G, BS, d = k_cache.shape[1], k_cache.shape[2], k_cache.shape[3]
+    dv, dims = v_cache.shape[3], cs.shape[1]
+    Cq = q_out.shape[1]
+    for r in range(proj.shape[0]):
+        p = int(positions[r])
+        if p < 0:
+            continue
+        row = proj[r].float()
+        q_out[r] = _rot_pairs(row[q_col: q_col + Cq].view(-1, d), cs[p],
+                              dims).reshape(-1).to(q_out.dtype)
+        blk = int(block_table[int(row_seq[r]), p // BS])
+        k_cache[blk, :, p % BS] = _rot_pairs(
+            row[k_col: k_col + G * d].view(G, d), cs[p], dims).to(
+            k_cache.dtype)
+        v_cache[blk, :, p % BS] = proj[r, v_col: v_col + G * dv].view(G, dv)
+
+
+def router_corrected(idx, wts, logits, correction, top: int, groups: int,
+                     keep: int, best: int, scale: float,
+                     renorm: bool) -> None:
+    """See the kernel: -inf for the experts outside the kept runs, ties to
+    the lower index; further columns of idx and wts are left alone."""
+    T, E = logits.shape
+    s = torch.sigmoid(logits.float())
+    c = s + correction if correction.numel() else s
+    if groups > 0:
+        runs = c.view(T, groups, E // groups)
+        value = runs.topk(min(best, E // groups), -1).values.sum(-1)
+        kept = torch.sort(value, dim=-1, descending=True,
+                          stable=True).indices[:, :keep]
+        ok = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, kept, True)
+        c = torch.where(ok.repeat_interleave(E // groups, 1), c,
+                        torch.full_like(c, -float("inf")))
+    ix = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top]
+    w = s.gather(1, ix)
+    if renorm:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    wts[:, :top] = w * scale
+    idx[:, :top] = ix.to(idx.dtype)

@@ -1010,7 +1010,8 @@ def case_op_attention(device, dtype, d=8, BS=4, n=90, start=0):
             out, dd(q), dd(kc), dd(vc) if o["own"] else None,
             dd(slopes) if o["lin"] else None, dd(r1) if o["log"] else None,
             dd(r2) if o["log"] else None, pos, row_seq, bt, H, o["scale"],
-            o["softcap"], o["chunk"], o["window"], o["sink"], o["key_eps"])
+            o["softcap"], o["chunk"], o["window"],
+            dd(torch.zeros(H)) if o["sink"] else None, o["key_eps"])
         _close(out, want, dtype, f"rows {o}")
         if o["window"] or o["lin"] or o["own"] or \
                 not ops.masked_tiles_supported(dd(q), d, BS):
@@ -1019,10 +1020,11 @@ def case_op_attention(device, dtype, d=8, BS=4, n=90, start=0):
         qb = list(range(0, n - start, 32))
         out = torch.full((n - start, H * d), 9.0, dtype=act, device=device)
         ops.masked_attention_tiles(
-            out, dd(q), dd(kc), dd(r1) if o["log"] else None,
-            dd(r2) if o["log"] else None, bt, i32([n]), i32([[start, 0]]),
-            i32([0] * len(qb)), i32(qb), o["scale"], o["softcap"], o["chunk"],
-            o["sink"], o["key_eps"])
+            out, dd(q), dd(kc), None, dd(r1) if o["log"] else None,
+            dd(r2) if o["log"] else None,
+            dd(torch.zeros(H)) if o["sink"] else None, bt, i32([n]),
+            i32([[start, 0]]), i32([0] * len(qb)), i32(qb), o["scale"],
+            o["softcap"], o["chunk"], 0, o["key_eps"])
         _close(out, want, dtype, f"tiles {o}")
 
 
