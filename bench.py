@@ -31,12 +31,12 @@ COMPARE_SIZES = {
 
 
 def compare_families(args) -> None:
-    """Prefill and decode tokens/s of Lipedra, Rasesun, Dumovik, Bezizen or
-    Noridra and of Llama (or another family) through the same engine at equal sizes: same
-    width, head counts,
-    feed-forward size, layer count and vocabulary (Llama head_dim 128;
-    Lipedra two score maps of 64 and value rows of 128 — equal cache bytes
-    per token; Rasesun three state-space layers to one latent-attention
+    """Prefill and decode tokens/s of Lipedra, Rasesun, Dumovik, Bezizen,
+    Noridra or Senavik and of Llama (or another family) through the same
+    engine at equal sizes: same width, head counts, feed-forward size, layer
+    count and vocabulary (Llama head_dim 128; Lipedra two score maps of 64 and
+    value rows of 128 — equal cache bytes per token; Rasesun three
+    state-space layers to one latent-attention
     layer with a 1024-token window, every second feed-forward a mixture of
     16 table-routed experts, two active; Dumovik periods of chunk-local
     attention over 8192-token chunks, two linear-attention layers and latent
@@ -46,7 +46,10 @@ def compare_families(args) -> None:
     attention, a shared expert everywhere and every second feed-forward a
     mixture of 16 routed experts, two active; Noridra delta rule, attention
     over 8192-token chunks, selective scan and delta rule, every second
-    feed-forward a mixture of 16 routed experts, two active)."""
+    feed-forward a mixture of 16 routed experts, two active; Senavik three
+    layers of attention over a 1024-token window and four kept tokens to one
+    of latent attention, every second feed-forward a mixture of 16 routed
+    experts, two active)."""
     from kukeon_amd.engine.config import (EngineConfig, ModelConfig,
                                           SamplingParams)
     from kukeon_amd.engine.engine import LLMEngine
@@ -57,6 +60,7 @@ def compare_families(args) -> None:
     from kukeon_amd.models.lipedra import lipedra_bench
     from kukeon_amd.models.noridra import noridra_bench
     from kukeon_amd.models.rasesun import rasesun_bench
+    from kukeon_amd.models.senavik import senavik_bench
 
     device = args.device or ("cuda:0" if torch.cuda.is_available() else "cpu")
     on_gpu = device != "cpu"
@@ -94,6 +98,12 @@ def compare_families(args) -> None:
                                     experts=16 if on_gpu else 4,
                                     max_positions=2048,
                                     name=f"noridra-{size}")
+            elif fam == "senavik":
+                cfg = senavik_bench(width=W, layers=nl, heads=hq,
+                                    kv_heads=hk, ff=ff, vocab=vocab,
+                                    window=1024 if on_gpu else 16,
+                                    experts=16 if on_gpu else 4,
+                                    name=f"senavik-{size}")
             elif fam == "dumovik":
                 cfg = dumovik_bench(width=W, layers=nl, heads=hq,
                                     kv_heads=hk, ff=ff, vocab=vocab,
@@ -188,12 +198,12 @@ def main() -> None:
                          "Llama at equal layer sizes (random weights)")
     ap.add_argument("--compare-family", default="lipedra",
                     choices=["lipedra", "rasesun", "dumovik", "bezizen",
-                             "noridra"],
+                             "noridra", "senavik"],
                     help="with --compare-families: the family that runs "
                          "beside Llama")
     ap.add_argument("--compare-against", default="llama",
                     choices=["llama", "lipedra", "rasesun", "dumovik",
-                             "bezizen"],
+                             "bezizen", "noridra"],
                     help="with --compare-families: the family it runs "
                          "beside (default Llama)")
     ap.add_argument("--compare-sizes", default="2k,4k,8k",

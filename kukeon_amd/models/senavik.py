@@ -131,15 +131,16 @@ def senavik_bench(width=4096, layers=8, heads=32, kv_heads=8, ff=14336,
                   vocab=128256, window=1024, keep_first=4, experts=16, top=2,
                   name="senavik-8b-like") -> SenavikConfig:
     """A layer stack at real-model sizes (random weights) for throughput
-    runs, in periods of four layers: three of windowed attention (heads of
-    128, half of a head rotated) and one of latent attention (heads of
-    128 + 64, a 512-wide latent, a query latent of 3/8 of the width);
+    runs, in periods of four layers (a shorter stack ends like one): three of
+    windowed attention (heads of 128, half of a head rotated) and one of
+    latent attention (heads of 128 + 64, a 512-wide latent, a query latent of
+    3/8 of the width);
     feed-forwards alternate between dense and routed experts of the same
     active size, the experts in four groups of which two are kept."""
     hd = 128 if width >= 1024 else 32
     ls = []
     for i in range(layers):
-        if i % 4 == 3:
+        if i % 4 == 3 or (layers < 4 and i == layers - 1 > 0):
             kind = "latent_attention"
             mix = LatentAttnCfg(
                 heads=heads, dim=128, rot_dim=64, vdim=128,

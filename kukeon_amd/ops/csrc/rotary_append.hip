@@ -9,25 +9,23 @@
 
 namespace kukeon {
 
-// VEC: a thread owns 8 entries of one head (16-byte accesses); otherwise one
-// entry, reading its partner besides.
+// blockIdx.x = row, the row's pieces over blockIdx.y and the threads. VEC: a
+// piece is 8 entries of one head (16-byte accesses); otherwise one entry, read
+// together with its partner.
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void rotary_append_kernel(
     T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
     const T* __restrict__ proj, long ldp, long q_col, long k_col, long v_col,
     const float* __restrict__ cs, int cs_rows, int dims,
     const int* __restrict__ positions, const int* __restrict__ row_seq,
-    const int* __restrict__ block_table, int max_blocks, long rows, int H,
-    int G, int d, int dv, int BS) {
+    const int* __restrict__ block_table, int max_blocks, int H, int G, int d,
+    int dv, int BS) {
   constexpr int N = VEC ? 8 : 1;
   const int Cq = H * d, Ck = G * d, Cv = G * dv;
-  const int per = (Cq + Ck + Cv) / N;
-  const long unit = (long)blockIdx.x * blockDim.x + threadIdx.x;
-  const long r = unit / per;
-  if (r >= rows) return;
+  const long r = blockIdx.x;
   const int p = positions[r];
-  if (p < 0) return;
-  int c = (int)(unit - r * per) * N;
+  int c = (int)(blockIdx.y * blockDim.x + threadIdx.x) * N;
+  if (p < 0 || c >= Cq + Ck + Cv) return;
   const T* row = proj + r * ldp;
   const T* src;
   T* dst;
@@ -129,10 +127,10 @@ void rotary_append(torch::Tensor q_out, torch::Tensor k_cache,
                    aligned16(q_out.data_ptr()) &&
                    aligned16(k_cache.data_ptr()) &&
                    aligned16(v_cache.data_ptr());
-  const long per = (long)H * d + (long)G * (d + dv);
-  const long threads = rows * (vec ? per / 8 : per);
+  const long per = ((long)H * d + (long)G * (d + dv)) / (vec ? 8 : 1);
+  TORCH_CHECK(per <= 65535L * 256);
   auto stream = c10::hip::getCurrentHIPStream().stream();
-  dim3 grid((unsigned)((threads + 255) / 256));
+  dim3 grid((unsigned)rows, (unsigned)((per + 255) / 256));
 #define KK_ARGS reinterpret_cast<T*>(q_out.data_ptr()),                        \
         reinterpret_cast<T*>(k_cache.data_ptr()),                              \
         reinterpret_cast<T*>(v_cache.data_ptr()),                              \
@@ -140,7 +138,7 @@ void rotary_append(torch::Tensor q_out, torch::Tensor k_cache,
         (long)q_col, (long)k_col, (long)v_col, cs.data_ptr<float>(),           \
         (int)cs.size(0), dims, positions.data_ptr<int>(),                      \
         row_seq.data_ptr<int>(), block_table.data_ptr<int>(),                  \
-        (int)block_table.size(1), rows, H, G, d, dv, BS
+        (int)block_table.size(1), H, G, d, dv, BS
   KK_DISPATCH_ACT(proj, {
     if (vec) rotary_append_kernel<T, true><<<grid, 256, 0, stream>>>(KK_ARGS);
     else rotary_append_kernel<T, false><<<grid, 256, 0, stream>>>(KK_ARGS);

@@ -242,9 +242,62 @@ DEV_INLINE int wave_argmax(float v, int i) {
   return i;
 }
 
-// One wave per row, experts over the lanes. In LDS: scores s [E], choice
-// scores c [E], run scores [groups]. -inf marks what cannot be chosen (any
-// more); a NaN logit counts as a score of 0 and the lowest choice score.
+// Score and choice score of a logit: a NaN counts as a score of 0 and the lowest
+// choice score, and no choice score is -inf, which marks what cannot be chosen.
+DEV_INLINE void corrected_score(float z, float corr, float& s, float& c) {
+  s = 1.0f / (1.0f + expf(-z));
+  c = s + corr;
+  c = c == c ? fmaxf(c, -3.0e38f) : -3.0e38f;
+  s = s == s ? s : 0.f;
+}
+
+// Up to 64 experts: one wave per row, lane = expert, everything by lane moves.
+// An expert's rank is the number of experts ahead of it (larger, or equal with
+// a lower index); ranks below `top` are the choice, in order.
+__global__ __launch_bounds__(256) void router_corrected_wave_kernel(
+    int* __restrict__ idx, float* __restrict__ wts, long ldi, long ldw,
+    const float* __restrict__ logits, long ldz,
+    const float* __restrict__ correction, long rows, int E, int top, int groups,
+    int keep, int best, float scale, int renorm) {
+  const long t = (long)blockIdx.x * 4 + threadIdx.x / WAVE;
+  if (t >= rows) return;                 // a whole wave
+  const int e = threadIdx.x & (WAVE - 1);
+  float s = 0.f, c = -INFINITY;
+  if (e < E)
+    corrected_score(logits[t * ldz + e], correction ? correction[e] : 0.f, s,
+                    c);
+  if (groups > 0) {
+    const int per = E / groups;
+    const int g = e / per;               // lanes past E are in no run
+    float a = -INFINITY, b = -INFINITY;  // the run's two largest
+    for (int i = 0; i < per; ++i) {
+      const float v = __shfl(c, min(g * per + i, WAVE - 1), WAVE);
+      b = fmaxf(b, fminf(a, v));
+      a = fmaxf(a, v);
+    }
+    const float gv = fmaxf(best > 1 && per > 1 ? a + b : a, -3.0e38f);
+    int rank = 0;
+    for (int o = 0; o < groups; ++o) {
+      const float v = __shfl(gv, o * per, WAVE);
+      rank += v > gv || (v == gv && o < g);
+    }
+    if (rank >= keep || e >= E) c = -INFINITY;
+  }
+  int rank = 0;
+  for (int o = 0; o < E; ++o) {
+    const float v = __shfl(c, o, WAVE);
+    rank += v > c || (v == c && o < e);
+  }
+  const bool chosen = e < E && rank < top;
+  const float sum = wave_sum(chosen ? s : 0.f);
+  if (chosen) {
+    idx[t * ldi + rank] = e;
+    wts[t * ldw + rank] = s * (renorm ? scale / (sum + 1e-20f) : scale);
+  }
+}
+
+// More experts: one wave per row, the experts in turns over the lanes. In LDS:
+// scores s [E], choice scores c [E], run scores [groups].
 __global__ __launch_bounds__(64) void router_corrected_kernel(
     int* __restrict__ idx, float* __restrict__ wts, long ldi, long ldw,
     const float* __restrict__ logits, long ldz,
@@ -258,10 +311,10 @@ __global__ __launch_bounds__(64) void router_corrected_kernel(
   const int lane = threadIdx.x;
   const float* z = logits + t * ldz;
   for (int e = lane; e < E; e += WAVE) {
-    const float sc = 1.0f / (1.0f + expf(-z[e]));
-    const float ch = correction ? sc + correction[e] : sc;
-    s[e] = sc == sc ? sc : 0.f;
-    c[e] = ch == ch ? fmaxf(ch, -3.0e38f) : -3.0e38f;
+    float sc, ch;
+    corrected_score(z[e], correction ? correction[e] : 0.f, sc, ch);
+    s[e] = sc;
+    c[e] = ch;
   }
   __syncthreads();
   if (groups > 0) {
@@ -341,6 +394,16 @@ void router_corrected(torch::Tensor idx, torch::Tensor wts,
   TORCH_CHECK(lds <= 60 * 1024, "router_corrected: too many experts");
   if (rows == 0) return;
   auto stream = c10::hip::getCurrentHIPStream().stream();
+  if (E <= WAVE) {
+    router_corrected_wave_kernel<<<dim3((unsigned)((rows + 3) / 4)), 256, 0,
+                                   stream>>>(
+        idx.data_ptr<int>(), wts.data_ptr<float>(), (long)idx.stride(0),
+        (long)wts.stride(0), logits.data_ptr<float>(), (long)logits.stride(0),
+        corr ? correction.data_ptr<float>() : nullptr, rows, E, (int)top,
+        (int)groups, (int)keep, (int)best, (float)scale, (int)renorm);
+    HIP_CHECK_KERNEL();
+    return;
+  }
   router_corrected_kernel<<<dim3((unsigned)rows), 64, lds, stream>>>(
       idx.data_ptr<int>(), wts.data_ptr<float>(), (long)idx.stride(0),
       (long)wts.stride(0), logits.data_ptr<float>(), (long)logits.stride(0),
